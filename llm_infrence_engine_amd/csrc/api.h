@@ -6,8 +6,8 @@
 
 extern "C" {
 
-int ms_embed(const int* ids, const void* table, float* out, int n_tokens, int hidden, float scale, int dtype,
-             hipStream_t stream);
+int ms_embed(const int* ids, const void* table, float* out, int n_tokens, int hidden, int copies, float scale, int dtype,
+             hipStream_t stream);     // out [n_tokens, copies, hidden], the copies all alike
 
 int ms_rms_norm(float* x, const void* delta, int delta_dtype, int n_partials, long long partial_stride,
                 const float* weight, const int* rows, void* out, int n_rows, int hidden, float eps, int write_back,
@@ -187,16 +187,19 @@ int ms_xielu(const void* x, const float* pq, void* out, long long total, int dty
 
 // ---- attention through a latent (csrc/latent_attention.hip); strides in elements
 int ms_head_matmul(const void* in, long long in_tok, long long in_head, const void* M, void* out, long long out_tok,
-                   long long out_head, const void* gate, long long gate_tok, int n_tokens, int heads, int I, int J,
-                   int dtype, int out_dtype, hipStream_t stream);
+                   long long out_head, const void* gate, long long gate_tok, int gate_w, int n_tokens, int heads, int I,
+                   int J, int dtype, int out_dtype, hipStream_t stream);    // gate_w: numbers a head, J or 1
+// the same on the matrix cores (csrc/head_matmul_mfma.hip): bfloat16, maps transposed [heads, J, I], I a multiple of 32
+int ms_head_matmul_mfma(const void* in, long long in_tok, long long in_head, const void* Mt, void* out, long long out_tok,
+                        long long out_head, const void* gate, long long gate_tok, int gate_w, int n_tokens, int heads, int I,
+                        int J, hipStream_t stream);
 int ms_rms_norm_rows(const void* in, long long in_stride, const float* weight, void* out, long long out_stride, int n_rows,
                      int width, float eps, int dtype, hipStream_t stream);
-int ms_rotary_pairs(const void* src, long long src_tok, long long src_head, void* dst, long long dst_tok,
-                    long long dst_head, const int* positions, const float* inv_freq, int n_tokens, int heads, int width,
-                    int dims, int dtype, hipStream_t stream);
-int ms_latent_kv_store(const void* kv, long long kv_stride, const float* norm_w, float eps, const int* positions,
-                       const float* inv_freq, const int* slots, void* c_pages, void* r_pages, void* ct_pages, int page_size,
-                       int n_tokens, int C, int R, int dims, int dtype, hipStream_t stream);
+int ms_latent_prepare(const void* kv, long long kv_stride, const float* norm_w, float eps, const int* positions,
+                      const float* inv_freq, float gain, int half, const int* slots, void* c_pages, void* r_pages,
+                      void* ct_pages, int page_size, const void* q_src, long long qs_tok, long long qs_head, void* q_dst,
+                      long long qd_tok, long long qd_head, int n_tokens, int heads, int C, int R, int dims, int dtype,
+                      hipStream_t stream);
 int ms_latent_attention(const void* q, long long q_tok, long long q_head, const void* c_pages, const void* r_pages,
                         const int* block_table, int table_stride, const int* table_rows, const int* n_live_tokens,
                         const int* token_req, const int* positions, const float* sink, void* out, long long out_tok,
@@ -209,7 +212,8 @@ int ms_latent_attention_mfma(const void* q, long long q_tok, long long q_head, c
                              const void* ct_pages, const int* block_table, int table_stride, const int* table_rows,
                              const int* q_start, const int* context_lens, const float* sink, void* out, long long out_tok,
                              long long out_head, int n_requests, int max_q_len, int heads, int C, int R, int page_size,
-                             long long num_pages, float scale, int window, hipStream_t stream);
+                             long long num_pages, float scale, int window, int splits, int n_tokens, float* part_o,
+                             float* part_ml, hipStream_t stream);
 
 // ---- layers that normalise a sublayer's output before it joins the residual stream (csrc/residual_norm.hip)
 // x += w_post * rms_norm(y); then, if out is not null, out = w_next * rms_norm(x).  y [n, hidden] in y_dtype (rows y_stride
@@ -237,10 +241,12 @@ int ms_selective_scan(const void* x, long long x_stride, const float* dt_in, con
 
 // ---- routed experts (csrc/experts.hip)
 int ms_gelu(const void* x, void* out, long long total, int dtype, hipStream_t stream);
+int ms_relu2(const void* x, void* out, long long total, int dtype, hipStream_t stream);
 // softmax over logits[n, :n_out] (rows ld apart; sigmoid_scores: each logit's own sigmoid instead), the `top` largest of
-// score + correction: ids / weights [n, top]
+// score + correction: ids / weights [n, top]; groups > 0: among the outputs of the `keep` best of so many equal groups of
+// neighbours; normalise: weights divided by their sum
 int ms_moe_route(const float* logits, long long ld, const float* correction, int n_tokens, int n_out, int top, int* ids,
-                 float* weights, int sigmoid_scores, hipStream_t stream);
+                 float* weights, int sigmoid_scores, int groups, int keep, int normalise, hipStream_t stream);
 int ms_moe_tile_rows();
 int ms_moe_wide_tile_rows();
 // rows [tiles * tile] and tile_expert [tiles] from ids [n_items]; ids >= n_experts take no row; tile: ms_moe_tile_rows()
@@ -262,7 +268,7 @@ int ms_grouped_gemm(const void* in, long long in_stride, const void* w, const in
                     int dtype, int out_dtype, hipStream_t stream);
 int ms_moe_combine(const float* part, const int* ids, const float* weights, const void* h, long long h_stride,
                    const void* shared, int shared_dtype, const float* gate, long long gate_stride, float* out,
-                   int n_tokens, int top, int n_experts, int hidden, int dtype, hipStream_t stream);   // weights null: all 1
+                   int n_tokens, int top, int n_experts, int hidden, int dtype, hipStream_t stream);   // weights null: all 1; gate null: shared added as it is
 
 // ---- layer norm and the gate of a token's side input (csrc/layer_norm.hip)
 int ms_layer_norm(float* x, const void* delta, int delta_dtype, const float* dscale, const float* w, const float* b, const int* rows,
@@ -296,9 +302,14 @@ int ms_pooled_attention_mfma(const void* q, long long q_stride, const void* k_pa
                              const float* turn_back, void* out, long long out_stride, int n_requests, int n_tokens,
                              int max_q_len, int num_heads, int num_kv_heads, int head_dim, int page_size, float scale,
                              int window, int pool, hipStream_t stream);
+// ---- a residual stream made of several copies that every sublayer reads and writes through numbers of its own (csrc/streams.hip)
+int ms_streams_max();
+int ms_streams(float* x, const void* base, int base_dtype, const float* part, const float* part_w, int top, const float* mix,
+               const float* b, const float* a, int norm, const float* w, const float* bias, float eps, const int* rows,
+               void* out, int out_dtype, int n_rows, int S, int W, int write_back, hipStream_t stream);
 // ---- gated activations (csrc/glu.hip)
-int ms_clamped_glu(const void* gu, long long in_stride, void* out, long long out_stride, int n_rows, int F, float limit,
-                   float alpha, int dtype, hipStream_t stream);
+int ms_clamped_glu(const void* gu, long long in_stride, const int* row_item, void* out, long long out_stride, int n_rows,
+                   int F, float limit, float alpha, int dtype, hipStream_t stream);
 int ms_scaled_swiglu(const void* gu, long long in_stride, const float* factor, const int* row_item, void* out,
                      long long out_stride, int n_rows, int F, int dtype, hipStream_t stream);
 int ms_gelu_tanh_glu(const void* gu, long long in_stride, void* out, long long out_stride, int n_rows, int F, int dtype,

@@ -7,23 +7,26 @@
 #include <algorithm>
 
 // ------------------------------------------------------------------------------------------------
-// out[n, :] = float(table[ids[n], :]) * scale
+// out[n, c, :] = float(table[ids[n], :]) * scale for every c < copies
 template <typename T>
 __global__ void embed_kernel(const int* __restrict__ ids, const T* __restrict__ table, float* __restrict__ out, int H,
-                             float scale) {
+                             int copies, float scale) {
   const int n = blockIdx.x;
   const T* row = table + (size_t)ids[n] * H;
-  float* o = out + (size_t)n * H;
-  for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = to_float(row[i]) * scale;
+  float* o = out + (size_t)n * copies * H;
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    const float v = to_float(row[i]) * scale;
+    for (int c = 0; c < copies; ++c) o[(size_t)c * H + i] = v;
+  }
 }
 
-extern "C" int ms_embed(const int* ids, const void* table, float* out, int n_tokens, int hidden, float scale, int dtype,
-                        hipStream_t stream) {
+extern "C" int ms_embed(const int* ids, const void* table, float* out, int n_tokens, int hidden, int copies, float scale,
+                        int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
-  if (hidden <= 0) return MS_BAD_ARG;
+  if (hidden <= 0 || copies <= 0) return MS_BAD_ARG;
   dim3 grid(n_tokens), block(256);
-  if (dtype == MS_F32) embed_kernel<float><<<grid, block, 0, stream>>>(ids, (const float*)table, out, hidden, scale);
-  else if (dtype == MS_BF16) embed_kernel<bf16><<<grid, block, 0, stream>>>(ids, (const bf16*)table, out, hidden, scale);
+  if (dtype == MS_F32) embed_kernel<float><<<grid, block, 0, stream>>>(ids, (const float*)table, out, hidden, copies, scale);
+  else if (dtype == MS_BF16) embed_kernel<bf16><<<grid, block, 0, stream>>>(ids, (const bf16*)table, out, hidden, copies, scale);
   else return MS_BAD_ARG;
   return ms_launch_status();
 }

@@ -1,10 +1,11 @@
 // Kernels of a feed-forward made of routed experts, all driven by device data so that a step can be captured:
-//   route    per token: softmax over the router's outputs, the `top` largest of (score + correction), their scores
+//   route    per token: softmax over the router's outputs, the `top` largest of (score + correction), their scores;
+//            optionally inside the best groups of neighbouring outputs only, and with the scores divided by their sum
 //   align    rows (token, choice) grouped by expert into tiles of TILE rows, each tile of one expert
 //   grouped  out[row] = act(W[expert of the row's tile] . in[row]) for every tile, gathered / scattered by the rows' list
 //   combine  out[n] = sum_j weight[n, j] * (expert j's row, or the token's input for an identity expert)
-//                     (+ sigmoid(gate[n]) * shared[n])
-// and the exact gelu, z/2 (1 + erf(z / sqrt 2)).  Router scores, weights and all sums are float.
+//                     (+ sigmoid(gate[n]) * shared[n], or + shared[n])
+// and two activations: the exact gelu, z/2 (1 + erf(z / sqrt 2)), and the square of relu.  Router scores, weights and all sums are float.
 #include "common.h"
 #include "api.h"
 
@@ -15,8 +16,13 @@ constexpr int ROUTE_MAX_TOP = 32;
 
 __device__ __forceinline__ float gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752440f)); }
 
-template <typename T>
-__global__ void gelu_kernel(const T* __restrict__ x, T* __restrict__ out, size_t total) {
+template <bool RELU2> __device__ __forceinline__ float act_of(float z) {
+  if (RELU2) { const float r = fmaxf(z, 0.f); return r * r; }
+  return gelu_erf(z);
+}
+
+template <typename T, bool RELU2>
+__global__ void act_kernel(const T* __restrict__ x, T* __restrict__ out, size_t total) {
   constexpr int V = 16 / sizeof(T);     // values in 16 bytes
   struct alignas(16) Pack { T v[V]; };
   const size_t stride = (size_t)gridDim.x * blockDim.x;
@@ -24,18 +30,22 @@ __global__ void gelu_kernel(const T* __restrict__ x, T* __restrict__ out, size_t
   for (size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < packs; i += stride) {
     Pack p = reinterpret_cast<const Pack*>(x)[i];
 #pragma unroll
-    for (int j = 0; j < V; ++j) p.v[j] = from_float<T>(gelu_erf(to_float(p.v[j])));
+    for (int j = 0; j < V; ++j) p.v[j] = from_float<T>(act_of<RELU2>(to_float(p.v[j])));
     reinterpret_cast<Pack*>(out)[i] = p;
   }
   for (size_t i = packs * V + (size_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += stride)
-    out[i] = from_float<T>(gelu_erf(to_float(x[i])));
+    out[i] = from_float<T>(act_of<RELU2>(to_float(x[i])));
 }
 
 // One wave per token.  Ties go to the lower index.  sigmoid_scores: every score is the sigmoid of its own logit
-// instead of the softmax over all of them.
+// instead of the softmax over all of them.  groups > 0: the outputs form that many equal groups of neighbours, a group
+// counts as its largest (score + correction), and only outputs of the `keep` best groups can be chosen.  normalise: the
+// chosen outputs' scores are divided by (their sum + 1e-20).
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __restrict__ correction, int n_tokens,
-                 int n_out, int top, int* __restrict__ ids, float* __restrict__ weights, int sigmoid_scores) {
+                 int n_out, int top, int* __restrict__ ids, float* __restrict__ weights, int sigmoid_scores, int groups,
+                 int keep, int normalise) {
+  extern __shared__ float s_choice[];     // with groups: [waves][n_out + groups] (score + correction, then the groups' maxima)
   const int lane = threadIdx.x & (MS_WAVE - 1);
   const int n = blockIdx.x * (blockDim.x / MS_WAVE) + threadIdx.x / MS_WAVE;
   if (n >= n_tokens) return;
@@ -64,6 +74,39 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
     s[i] *= inv;
     c[i] = e < n_out ? s[i] + (correction ? correction[e] : 0.f) : -INFINITY;
   }
+  if (groups > 0) {
+    // the wave works in its own stretch of LDS: what its lanes wrote is there for its lanes to read, in order
+    float* choice = s_choice + (size_t)(threadIdx.x / MS_WAVE) * (n_out + groups);
+    float* best = choice + n_out;
+    const int size = n_out / groups;
+#pragma unroll
+    for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
+      if (lane + i * MS_WAVE < n_out) choice[lane + i * MS_WAVE] = c[i];
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    for (int g = lane; g < groups; g += MS_WAVE) {
+      float m = -INFINITY;
+      for (int i = 0; i < size; ++i) m = fmaxf(m, choice[g * size + i]);
+      best[g] = m;
+    }
+    __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    // an output stays when fewer than `keep` groups come before its own (larger, or equal and earlier)
+#pragma unroll
+    for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
+      const int e = lane + i * MS_WAVE;
+      if (e >= n_out) continue;
+      const int mine = e / size;
+      const float m = best[mine];
+      int before = 0;
+      for (int g = 0; g < groups; ++g) {
+        const float o = best[g];
+        if (o > m || (o == m && g < mine)) ++before;
+      }
+      if (before >= keep) c[i] = -INFINITY;
+    }
+  }
+  float my_weight = 0.f, total = 0.f;
   for (int j = 0; j < top; ++j) {
     float bv = -INFINITY, bs = 0.f;
     int be = 0x7fffffff;
@@ -78,11 +121,14 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
       const int oe = __shfl_xor(be, o, MS_WAVE);
       if (ov > bv || (ov == bv && oe < be)) { bv = ov; be = oe; bs = os; }
     }
-    if (lane == 0) { ids[(size_t)n * top + j] = be; weights[(size_t)n * top + j] = bs; }
+    if (lane == 0) ids[(size_t)n * top + j] = be;
+    if (lane == j) my_weight = bs;
+    total += bs;
 #pragma unroll
     for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
       if (lane + i * MS_WAVE == be) c[i] = -INFINITY;
   }
+  if (lane < top) weights[(size_t)n * top + lane] = normalise ? my_weight / (total + 1e-20f) : my_weight;
 }
 
 // One block.  rows[cap] (cap = tiles * tile): for every tile its rows' flat index n * top + j, or -1; tile_expert[tiles]:
@@ -368,6 +414,7 @@ grouped_gemm_mfma_wide_kernel(const bf16* __restrict__ in, size_t in_stride, con
 }
 
 // out[n, :] = sum_j weights[n, j] * (ids[n, j] < n_experts ? part[n * top + j, :] : h[n, :]) + sigmoid(gate[n]) * shared[n, :]
+// (gate null: + shared[n, :])
 template <typename T, typename TS>
 __global__ void __launch_bounds__(256)
 moe_combine_kernel(const float* __restrict__ part, const int* __restrict__ ids, const float* __restrict__ weights,
@@ -381,8 +428,8 @@ moe_combine_kernel(const float* __restrict__ part, const int* __restrict__ ids, 
     s_w[threadIdx.x] = weights ? weights[(size_t)n * top + threadIdx.x] : 1.0f;
   }
   __syncthreads();
-  float g = 0.f;
-  if (shared) { const float z = gate[(size_t)n * gate_stride]; g = 1.0f / (1.0f + expf(-z)); }
+  float g = 1.f;
+  if (shared && gate) { const float z = gate[(size_t)n * gate_stride]; g = 1.0f / (1.0f + expf(-z)); }
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
     float acc = 0.f;
     for (int j = 0; j < top; ++j) {
@@ -396,23 +443,35 @@ moe_combine_kernel(const float* __restrict__ part, const int* __restrict__ ids, 
 
 }  // namespace
 
-extern "C" int ms_gelu(const void* x, void* out, long long total, int dtype, hipStream_t stream) {
+template <bool RELU2>
+static int launch_act(const void* x, void* out, long long total, int dtype, hipStream_t stream) {
   if (total <= 0) return MS_OK;
   int blocks = (int)((total / 4 + 255) / 256) + 1;
   if (blocks > 8192) blocks = 8192;
-  if (dtype == MS_F32) gelu_kernel<float><<<blocks, 256, 0, stream>>>((const float*)x, (float*)out, (size_t)total);
-  else if (dtype == MS_BF16) gelu_kernel<bf16><<<blocks, 256, 0, stream>>>((const bf16*)x, (bf16*)out, (size_t)total);
+  if (dtype == MS_F32) act_kernel<float, RELU2><<<blocks, 256, 0, stream>>>((const float*)x, (float*)out, (size_t)total);
+  else if (dtype == MS_BF16) act_kernel<bf16, RELU2><<<blocks, 256, 0, stream>>>((const bf16*)x, (bf16*)out, (size_t)total);
   else return MS_BAD_ARG;
   return ms_launch_status();
 }
 
+extern "C" int ms_gelu(const void* x, void* out, long long total, int dtype, hipStream_t stream) {
+  return launch_act<false>(x, out, total, dtype, stream);
+}
+
+extern "C" int ms_relu2(const void* x, void* out, long long total, int dtype, hipStream_t stream) {
+  return launch_act<true>(x, out, total, dtype, stream);
+}
+
 extern "C" int ms_moe_route(const float* logits, long long ld, const float* correction, int n_tokens, int n_out, int top,
-                            int* ids, float* weights, int sigmoid_scores, hipStream_t stream) {
+                            int* ids, float* weights, int sigmoid_scores, int groups, int keep, int normalise,
+                            hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
-  if (n_out <= 0 || top <= 0 || top > n_out) return MS_BAD_ARG;
+  if (n_out <= 0 || top <= 0 || top > n_out || groups < 0) return MS_BAD_ARG;
+  if (groups > 0 && (n_out % groups || keep <= 0 || keep > groups || top > keep * (n_out / groups))) return MS_BAD_ARG;
   if (n_out > ROUTE_MAX_PER_LANE * MS_WAVE || top > ROUTE_MAX_TOP) return MS_UNSUPPORTED;
-  moe_route_kernel<<<(n_tokens + 3) / 4, 256, 0, stream>>>(logits, (size_t)ld, correction, n_tokens, n_out, top, ids,
-                                                           weights, sigmoid_scores);
+  const size_t lds = groups > 0 ? (size_t)4 * (n_out + groups) * sizeof(float) : 0;
+  moe_route_kernel<<<(n_tokens + 3) / 4, 256, lds, stream>>>(logits, (size_t)ld, correction, n_tokens, n_out, top, ids,
+                                                             weights, sigmoid_scores, groups, keep, normalise);
   return ms_launch_status();
 }
 
@@ -491,7 +550,7 @@ extern "C" int ms_moe_combine(const float* part, const int* ids, const float* we
                               const void* shared, int shared_dtype, const float* gate, long long gate_stride, float* out,
                               int n_tokens, int top, int n_experts, int hidden, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
-  if (top <= 0 || top > ROUTE_MAX_TOP || hidden <= 0 || (shared != nullptr && gate == nullptr)) return MS_BAD_ARG;
+  if (top <= 0 || top > ROUTE_MAX_TOP || hidden <= 0) return MS_BAD_ARG;
   dim3 grid(n_tokens), block(256);
 #define LAUNCH(T, TS)                                                                                                \
   moe_combine_kernel<T, TS><<<grid, block, 0, stream>>>(part, ids, weights, (const T*)h, (size_t)h_stride,           \

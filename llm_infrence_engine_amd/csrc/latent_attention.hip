@@ -4,8 +4,8 @@
 // query and to the output and the attention itself runs over the cached latents alone, as one key/value "head"
 // that every query head reads.
 //   ms_head_matmul      out[n, h, :] = in[n, h, :] @ M[h]  (the two per-head maps), optionally gated
-//   ms_rotary_pairs     rotation of neighbouring pairs (2i, 2i+1) by position * inv_freq[i], copying the rest
-//   ms_latent_kv_store  RMS norm of the latent, rotation of the shared key part, both into their pages
+//   ms_latent_prepare   per token: RMS norm of the latent, rotation of the shared key part, both into their pages, and
+//                       the rotation of the query heads' rotated slices
 //   ms_latent_attention sliding-window softmax attention over the pages with a per-head sink in the denominator
 // Scores, softmax, norms and angles are float in every mode.
 #include "common.h"
@@ -16,7 +16,8 @@ namespace {
 __device__ __forceinline__ float sigmoid_f(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 // ------------------------------------------------------------------------------------------------
-// out[n, h, j] = sum_i in[n, h, i] * M[h, i, j] (* sigmoid(gate[n, h, j])).  A block owns TM tokens of one head and 64
+// out[n, h, j] = sum_i in[n, h, i] * M[h, i, j] (* sigmoid(gate[n, h, j]), or of one number per head: gate_w = J
+// or 1 numbers a head).  A block owns TM tokens of one head and 64
 // consecutive j; its four waves each take a quarter of the i (rows of M, read coalesced, eight in flight) and their
 // sums are added through LDS in wave order: the shape for few tokens (a decode step), where blocks are few and a
 // thread's walk over all the i would be the longest chain of the step.
@@ -26,7 +27,7 @@ template <typename T, typename TO, int TM>
 __global__ void __launch_bounds__(HM_WAVES * MS_WAVE)
 head_matmul_kernel(const T* __restrict__ in, size_t in_tok, size_t in_head, const T* __restrict__ M,
                    TO* __restrict__ out, size_t out_tok, size_t out_head, const T* __restrict__ gate,
-                   size_t gate_tok, int N, int I, int J) {
+                   size_t gate_tok, int gate_w, int N, int I, int J) {
   extern __shared__ __align__(16) float xs[];   // [I][TM], then [HM_WAVES - 1][TM][64] for the waves' sums
   float* part = xs + (size_t)I * TM;
   const int h = blockIdx.y, n0 = blockIdx.x * TM;
@@ -66,7 +67,7 @@ head_matmul_kernel(const T* __restrict__ in, size_t in_tok, size_t in_head, cons
     if (n0 + t >= N) break;
     float y = acc[t];
     for (int w = 0; w < HM_WAVES - 1; ++w) y += part[(w * TM + t) * MS_WAVE + lane];
-    if (gate) y *= sigmoid_f(to_float(gate[(size_t)(n0 + t) * gate_tok + (size_t)h * J + j]));
+    if (gate) y *= sigmoid_f(to_float(gate[(size_t)(n0 + t) * gate_tok + (size_t)h * gate_w + (gate_w > 1 ? j : 0)]));
     out[(size_t)(n0 + t) * out_tok + (size_t)h * out_head + j] = from_float<TO>(y);
   }
 }
@@ -78,7 +79,7 @@ constexpr int HM_TOKENS = 8;
 template <typename T, typename TO>
 __global__ void head_matmul_wide_kernel(const T* __restrict__ in, size_t in_tok, size_t in_head, const T* __restrict__ M,
                                         TO* __restrict__ out, size_t out_tok, size_t out_head, const T* __restrict__ gate,
-                                        size_t gate_tok, int N, int I, int J) {
+                                        size_t gate_tok, int gate_w, int N, int I, int J) {
   extern __shared__ __align__(16) float xs[];   // [I][HM_TOKENS]
   const int h = blockIdx.y, n0 = blockIdx.x * HM_TOKENS;
   const int j = blockIdx.z * blockDim.x + threadIdx.x;
@@ -104,36 +105,8 @@ __global__ void head_matmul_wide_kernel(const T* __restrict__ in, size_t in_tok,
   for (int t = 0; t < HM_TOKENS; ++t) {
     if (n0 + t >= N) break;
     float y = acc[t];
-    if (gate) y *= sigmoid_f(to_float(gate[(size_t)(n0 + t) * gate_tok + (size_t)h * J + j]));
+    if (gate) y *= sigmoid_f(to_float(gate[(size_t)(n0 + t) * gate_tok + (size_t)h * gate_w + (gate_w > 1 ? j : 0)]));
     out[(size_t)(n0 + t) * out_tok + (size_t)h * out_head + j] = from_float<TO>(y);
-  }
-}
-
-// ------------------------------------------------------------------------------------------------
-// dst[n, h, 0:width] = src[n, h, 0:width] with the first `dims` entries turned pair by pair:
-// (u, v) = entries (2i, 2i+1) -> (u cos a - v sin a, v cos a + u sin a), a = float(position) * inv_freq[i].
-template <typename T>
-__global__ void rotary_pairs_kernel(const T* __restrict__ src, size_t src_tok, size_t src_head, T* __restrict__ dst,
-                                    size_t dst_tok, size_t dst_head, const int* __restrict__ positions,
-                                    const float* __restrict__ inv_freq, int heads, int width, int dims) {
-  const int n = blockIdx.x;
-  const float pos = (float)positions[n];
-  const int half = width / 2 + (width & 1);   // pairs, and a last single entry if the width is odd
-  for (int e = threadIdx.x; e < heads * half; e += blockDim.x) {
-    const int h = e / half, i = e - h * half;
-    const T* s = src + (size_t)n * src_tok + (size_t)h * src_head;
-    T* d = dst + (size_t)n * dst_tok + (size_t)h * dst_head;
-    if (2 * i + 1 >= width) { d[2 * i] = s[2 * i]; continue; }
-    const float u = to_float(s[2 * i]), v = to_float(s[2 * i + 1]);
-    if (2 * i + 1 < dims) {
-      float sn, cs;
-      sincosf(pos * inv_freq[i], &sn, &cs);
-      d[2 * i] = from_float<T>(u * cs - v * sn);
-      d[2 * i + 1] = from_float<T>(v * cs + u * sn);
-    } else {
-      d[2 * i] = s[2 * i];
-      d[2 * i + 1] = s[2 * i + 1];
-    }
   }
 }
 
@@ -153,15 +126,47 @@ __global__ void rms_norm_rows_kernel(const T* __restrict__ in, size_t in_stride,
 }
 
 // ------------------------------------------------------------------------------------------------
-// kv [N, C + R]: c = rms_norm(kv[:, :C]) * w -> latent pages at the token's slot; kv[:, C:] rotated -> key-part pages.
-// Pages are [page][slot][entry] with one head.
+// One block per token.  The first `dims` entries of a slice turn pair by pair, (u, v) -> gain (u cos a - v sin a,
+// v cos a + u sin a) with a = float(position) * inv_freq[i]: entries (2i, 2i + 1), or (i, i + dims / 2) with `half`; the
+// rest pass unchanged.  kv (may be null) [N, C + R]: c = rms_norm(kv[:, :C]) * w -> latent pages at the token's slot;
+// kv[:, C:] turned -> key-part pages (pages are [page][slot][entry] with one head).  q_src (may be null) [N, heads, R]:
+// every head's slice turned -> q_dst (which may be q_src).
 template <typename T>
-__global__ void latent_kv_store_kernel(const T* __restrict__ kv, size_t kv_stride, const float* __restrict__ w, float eps,
-                                       const int* __restrict__ positions, const float* __restrict__ inv_freq,
-                                       const int* __restrict__ slots, T* __restrict__ c_pages, T* __restrict__ r_pages,
-                                       T* __restrict__ ct_pages, int page_size, int C, int R, int dims) {
+__device__ __forceinline__ void turn_pair(const T* __restrict__ s, T* d, int i, int half, int pairs, const float* __restrict__ turn) {
+  const int iu = half ? i : 2 * i, iv = half ? i + pairs : 2 * i + 1;
+  const float u = to_float(s[iu]), v = to_float(s[iv]), cs = turn[2 * i], sn = turn[2 * i + 1];
+  d[iu] = from_float<T>(u * cs - v * sn);
+  d[iv] = from_float<T>(v * cs + u * sn);
+}
+
+template <typename T>
+__global__ void latent_prepare_kernel(const T* __restrict__ kv, size_t kv_stride, const float* __restrict__ w, float eps,
+                                      const int* __restrict__ positions, const float* __restrict__ inv_freq, float gain, int half,
+                                      const int* __restrict__ slots, T* __restrict__ c_pages, T* __restrict__ r_pages,
+                                      T* __restrict__ ct_pages, int page_size, const T* q_src, size_t qs_tok, size_t qs_head,
+                                      T* q_dst, size_t qd_tok, size_t qd_head, int heads, int C, int R, int dims) {
+  extern __shared__ __align__(16) float turn[];     // [dims / 2] pairs (cos, sin)
   __shared__ float red[16];
-  const int n = blockIdx.x;
+  const int n = blockIdx.x, pairs = dims / 2, rest = R - dims;
+  const float pos = (float)positions[n];
+  for (int i = threadIdx.x; i < pairs; i += blockDim.x) {
+    float sn, cs;
+    sincosf(pos * inv_freq[i], &sn, &cs);
+    turn[2 * i] = cs * gain;
+    turn[2 * i + 1] = sn * gain;
+  }
+  __syncthreads();
+  if (q_src) {
+    const int per = pairs + rest;
+    for (int e = threadIdx.x; e < heads * per; e += blockDim.x) {
+      const int h = e / per, i = e - h * per;
+      const T* s = q_src + (size_t)n * qs_tok + (size_t)h * qs_head;
+      T* d = q_dst + (size_t)n * qd_tok + (size_t)h * qd_head;
+      if (i < pairs) turn_pair(s, d, i, half, pairs, turn);
+      else d[dims + i - pairs] = s[dims + i - pairs];
+    }
+  }
+  if (!kv) return;
   const int slot = slots[n];
   if (slot < 0) return;        // uniform for the block: a token that stores nothing
   const T* x = kv + (size_t)n * kv_stride;
@@ -178,21 +183,11 @@ __global__ void latent_kv_store_kernel(const T* __restrict__ kv, size_t kv_strid
     cp[i] = v;
     if (tp) tp[(size_t)i * page_size] = v;
   }
-  const float pos = (float)positions[n];
   T* rp = r_pages + (size_t)slot * R;
   const T* xr = x + C;
-  for (int i = threadIdx.x; i < (R + 1) / 2; i += blockDim.x) {
-    if (2 * i + 1 >= R) { rp[2 * i] = xr[2 * i]; continue; }
-    const float u = to_float(xr[2 * i]), v = to_float(xr[2 * i + 1]);
-    if (2 * i + 1 < dims) {
-      float sn, cs;
-      sincosf(pos * inv_freq[i], &sn, &cs);
-      rp[2 * i] = from_float<T>(u * cs - v * sn);
-      rp[2 * i + 1] = from_float<T>(v * cs + u * sn);
-    } else {
-      rp[2 * i] = xr[2 * i];
-      rp[2 * i + 1] = xr[2 * i + 1];
-    }
+  for (int i = threadIdx.x; i < pairs + rest; i += blockDim.x) {
+    if (i < pairs) turn_pair(xr, rp, i, half, pairs, turn);
+    else rp[dims + i - pairs] = xr[dims + i - pairs];
   }
 }
 
@@ -277,17 +272,17 @@ latent_attention_kernel(const T* __restrict__ q, size_t q_tok, size_t q_head, co
 }  // namespace
 
 extern "C" int ms_head_matmul(const void* in, long long in_tok, long long in_head, const void* M, void* out,
-                              long long out_tok, long long out_head, const void* gate, long long gate_tok, int n_tokens,
-                              int heads, int I, int J, int dtype, int out_dtype, hipStream_t stream) {
+                              long long out_tok, long long out_head, const void* gate, long long gate_tok, int gate_w,
+                              int n_tokens, int heads, int I, int J, int dtype, int out_dtype, hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
-  if (heads <= 0 || I <= 0 || J <= 0) return MS_BAD_ARG;
+  if (heads <= 0 || I <= 0 || J <= 0 || (gate && gate_w != 1 && gate_w != J)) return MS_BAD_ARG;
   // float: always the one order of summation, whatever the step holds
   if (n_tokens > 64 || dtype == MS_F32) {
     const size_t lds = (size_t)I * HM_TOKENS * sizeof(float);
     if (lds > 65536 || heads > 65535) return MS_UNSUPPORTED;
     const int threads = J >= 256 ? 256 : ((J + MS_WAVE - 1) / MS_WAVE) * MS_WAVE;
     dim3 grid((n_tokens + HM_TOKENS - 1) / HM_TOKENS, heads, (J + threads - 1) / threads), block(threads);
-#define LAUNCH(T, TO) head_matmul_wide_kernel<T, TO><<<grid, block, lds, stream>>>((const T*)in, (size_t)in_tok, (size_t)in_head, (const T*)M, (TO*)out, (size_t)out_tok, (size_t)out_head, (const T*)gate, (size_t)gate_tok, n_tokens, I, J)
+#define LAUNCH(T, TO) head_matmul_wide_kernel<T, TO><<<grid, block, lds, stream>>>((const T*)in, (size_t)in_tok, (size_t)in_head, (const T*)M, (TO*)out, (size_t)out_tok, (size_t)out_head, (const T*)gate, (size_t)gate_tok, gate_w, n_tokens, I, J)
     if (dtype == MS_F32 && out_dtype == MS_F32) LAUNCH(float, float);
     else if (dtype == MS_BF16 && out_dtype == MS_BF16) LAUNCH(bf16, bf16);
     else if (dtype == MS_BF16 && out_dtype == MS_F32) LAUNCH(bf16, float);
@@ -299,7 +294,7 @@ extern "C" int ms_head_matmul(const void* in, long long in_tok, long long in_hea
   const size_t lds = ((size_t)I * tm + (size_t)(HM_WAVES - 1) * tm * MS_WAVE) * sizeof(float);
   if (lds > 65536 || heads > 65535 || (J + MS_WAVE - 1) / MS_WAVE > 65535) return MS_UNSUPPORTED;
   dim3 grid((n_tokens + tm - 1) / tm, heads, (J + MS_WAVE - 1) / MS_WAVE), block(HM_WAVES * MS_WAVE);
-#define LAUNCH(T, TO) head_matmul_kernel<T, TO, 8><<<grid, block, lds, stream>>>((const T*)in, (size_t)in_tok, (size_t)in_head, (const T*)M, (TO*)out, (size_t)out_tok, (size_t)out_head, (const T*)gate, (size_t)gate_tok, n_tokens, I, J)
+#define LAUNCH(T, TO) head_matmul_kernel<T, TO, 8><<<grid, block, lds, stream>>>((const T*)in, (size_t)in_tok, (size_t)in_head, (const T*)M, (TO*)out, (size_t)out_tok, (size_t)out_head, (const T*)gate, (size_t)gate_tok, gate_w, n_tokens, I, J)
   if (dtype == MS_F32 && out_dtype == MS_F32) LAUNCH(float, float);
   else if (dtype == MS_BF16 && out_dtype == MS_BF16) LAUNCH(bf16, bf16);
   else if (dtype == MS_BF16 && out_dtype == MS_F32) LAUNCH(bf16, float);
@@ -323,35 +318,24 @@ extern "C" int ms_rms_norm_rows(const void* in, long long in_stride, const float
   return ms_launch_status();
 }
 
-extern "C" int ms_rotary_pairs(const void* src, long long src_tok, long long src_head, void* dst, long long dst_tok,
-                               long long dst_head, const int* positions, const float* inv_freq, int n_tokens, int heads,
-                               int width, int dims, int dtype, hipStream_t stream) {
+// kv null: no store (norm_w, slots and the pages are not read); q_src null: no query slices.
+extern "C" int ms_latent_prepare(const void* kv, long long kv_stride, const float* norm_w, float eps, const int* positions,
+                                 const float* inv_freq, float gain, int half, const int* slots, void* c_pages, void* r_pages,
+                                 void* ct_pages, int page_size, const void* q_src, long long qs_tok, long long qs_head,
+                                 void* q_dst, long long qd_tok, long long qd_head, int n_tokens, int heads, int C, int R,
+                                 int dims, int dtype, hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
-  if (heads <= 0 || width <= 0 || dims < 0 || dims > width || dims % 2) return MS_BAD_ARG;
+  if (R <= 0 || dims < 0 || dims > R || dims % 2) return MS_BAD_ARG;
+  if (kv && (C <= 0 || page_size <= 0 || !norm_w || !slots || !c_pages || !r_pages)) return MS_BAD_ARG;
+  if (q_src && (heads <= 0 || !q_dst)) return MS_BAD_ARG;
+  const size_t lds = (size_t)dims * sizeof(float);
+  if (lds > 32768) return MS_UNSUPPORTED;
   dim3 grid(n_tokens), block(256);
-  if (dtype == MS_F32)
-    rotary_pairs_kernel<float><<<grid, block, 0, stream>>>((const float*)src, (size_t)src_tok, (size_t)src_head, (float*)dst,
-                                                           (size_t)dst_tok, (size_t)dst_head, positions, inv_freq, heads, width, dims);
-  else if (dtype == MS_BF16)
-    rotary_pairs_kernel<bf16><<<grid, block, 0, stream>>>((const bf16*)src, (size_t)src_tok, (size_t)src_head, (bf16*)dst,
-                                                          (size_t)dst_tok, (size_t)dst_head, positions, inv_freq, heads, width, dims);
+#define LAUNCH(T) latent_prepare_kernel<T><<<grid, block, lds, stream>>>((const T*)kv, (size_t)kv_stride, norm_w, eps, positions, inv_freq, gain, half, slots, (T*)c_pages, (T*)r_pages, (T*)ct_pages, page_size, (const T*)q_src, (size_t)qs_tok, (size_t)qs_head, (T*)q_dst, (size_t)qd_tok, (size_t)qd_head, heads, C, R, dims)
+  if (dtype == MS_F32) LAUNCH(float);
+  else if (dtype == MS_BF16) LAUNCH(bf16);
   else return MS_BAD_ARG;
-  return ms_launch_status();
-}
-
-extern "C" int ms_latent_kv_store(const void* kv, long long kv_stride, const float* norm_w, float eps, const int* positions,
-                                  const float* inv_freq, const int* slots, void* c_pages, void* r_pages, void* ct_pages,
-                                  int page_size, int n_tokens, int C, int R, int dims, int dtype, hipStream_t stream) {
-  if (n_tokens <= 0) return MS_OK;
-  if (C <= 0 || R <= 0 || dims < 0 || dims > R || dims % 2 || page_size <= 0) return MS_BAD_ARG;
-  dim3 grid(n_tokens), block(C >= 512 ? 256 : 128);
-  if (dtype == MS_F32)
-    latent_kv_store_kernel<float><<<grid, block, 0, stream>>>((const float*)kv, (size_t)kv_stride, norm_w, eps, positions, inv_freq,
-                                                              slots, (float*)c_pages, (float*)r_pages, (float*)ct_pages, page_size, C, R, dims);
-  else if (dtype == MS_BF16)
-    latent_kv_store_kernel<bf16><<<grid, block, 0, stream>>>((const bf16*)kv, (size_t)kv_stride, norm_w, eps, positions, inv_freq,
-                                                             slots, (bf16*)c_pages, (bf16*)r_pages, (bf16*)ct_pages, page_size, C, R, dims);
-  else return MS_BAD_ARG;
+#undef LAUNCH
   return ms_launch_status();
 }
 

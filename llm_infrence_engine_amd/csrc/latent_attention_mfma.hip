@@ -16,7 +16,9 @@
 // The sums of the exponentials come from one more product with ones (the bfloat16 values that weigh the latents).
 // Values past the last visible key are zeroed before use and pages past the context are never dereferenced.
 // Launch: grid (column tiles of the longest portion, requests); a block without a tile leaves at once, so the launch
-// depends on the step's number of requests and longest portion only.
+// depends on the step's number of requests and longest portion only.  A step of single tokens may spread a tile's key
+// blocks over several blocks (grid z, SPLIT): each leaves its accumulators with their maximum and sum, and
+// latent_combine_kernel adds a column's parts up in split order.
 #include "common.h"
 #include "api.h"
 
@@ -28,14 +30,15 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 constexpr int LM_WAVES = 4;
 
-template <int C, int R>
+template <int C, int R, bool SPLIT>
 __global__ void __launch_bounds__(LM_WAVES * MS_WAVE)
 latent_attention_mfma_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_head, const bf16* __restrict__ c_pages,
                              const bf16* __restrict__ r_pages, const bf16* __restrict__ ct_pages,
                              const int* __restrict__ block_table, int table_stride, const int* __restrict__ table_rows,
                              const int* __restrict__ q_start, const int* __restrict__ context_lens,
                              const float* __restrict__ sink, bf16* __restrict__ out, size_t out_tok, size_t out_head,
-                             int H, int page_size, float scale_log2e, int window) {
+                             int H, int page_size, float scale_log2e, int window, float* __restrict__ part_o,
+                             float* __restrict__ part_ml) {
   constexpr int KS_C = C / 32, KS_R = R / 32, CT = C / 16;
   __shared__ float sm_m[LM_WAVES][16], sm_l[LM_WAVES][16];
   __shared__ f32x4 sm_o[CT][MS_WAVE];
@@ -76,7 +79,14 @@ latent_attention_mfma_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_
 #pragma unroll
   for (int t = 0; t < CT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  for (int base = (key_lo / 32 + wave) * 32; base <= key_hi; base += 32 * LM_WAVES) {
+  // this block's key blocks of 32: all of the tile's, or (SPLIT) its share of them
+  int b_lo = key_lo / 32, b_hi = key_hi / 32;
+  if (SPLIT) {
+    const int share = (b_hi - b_lo + (int)gridDim.z) / (int)gridDim.z;     // rounded up
+    b_lo += (int)blockIdx.z * share;
+    b_hi = min(b_hi, b_lo + share - 1);
+  }
+  for (int base = (b_lo + wave) * 32; base <= b_hi * 32; base += 32 * LM_WAVES) {
     // the two 16-key halves of the block: a half lies in one page (pages hold a multiple of 16 keys)
     size_t row0[2];     // first key's row in the pools (page * page_size + offset); the null page past the context
 #pragma unroll
@@ -140,7 +150,8 @@ latent_attention_mfma_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_
     const bool tail = base + 31 > key_hi;
     const bf16* vp0 = ct_pages + (row0[0] / page_size) * (size_t)page_size * C + row0[0] % page_size + kq * 4;
     const bf16* vp1 = ct_pages + (row0[1] / page_size) * (size_t)page_size * C + row0[1] % page_size + kq * 4;
-    constexpr int VG = CT < 16 ? CT : 16;      // tiles of 16 entries whose values are asked for together
+    constexpr int VG = CT <= 16 ? CT : (CT % 16 ? 12 : 16);     // tiles of 16 entries whose values are asked for together
+    static_assert(CT % VG == 0, "the latent's tiles come in whole groups");
 #pragma unroll
     for (int t0 = 0; t0 < CT; t0 += VG) {
       bf16x4 va[VG], vb[VG];
@@ -196,6 +207,14 @@ latent_attention_mfma_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_
     __syncthreads();
   }
   if (wave != 0 || pos < 0) return;
+  if (SPLIT) {            // (a share without keys leaves m = -inf, l = 0 and zeros)
+    const size_t at = ((size_t)tok * H + head) * gridDim.z + blockIdx.z;
+    float* po = part_o + at * C + kq * 4;
+#pragma unroll
+    for (int t = 0; t < CT; ++t) *reinterpret_cast<f32x4*>(po + t * 16) = o[t];
+    if (kq == 0) { part_ml[2 * at] = m; part_ml[2 * at + 1] = l; }
+    return;
+  }
   if (sink) {             // the sink: one more term exp(sink) in the denominator, unscaled, with no value
     const float sk = sink[head] * 1.4426950408889634f;
     const float big = fmaxf(m, sk);
@@ -212,6 +231,34 @@ latent_attention_mfma_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_
 #pragma unroll
     for (int i = 0; i < 4; ++i) w[i] = (__bf16)(o[t][i] * inv);
     *reinterpret_cast<bf16x4*>(op + t * 16) = w;
+  }
+}
+
+// out[column] = sum over the splits of a column's parts, brought to one maximum, divided by their sums (and the sink's
+// term).  A block per (token, head); tokens of no request (from q_start[n_requests] on) are left alone.
+__global__ void __launch_bounds__(128)
+latent_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const int* __restrict__ q_start,
+                      int n_requests, const float* __restrict__ sink, bf16* __restrict__ out, size_t out_tok,
+                      size_t out_head, int H, int C, int splits) {
+  const int tok = blockIdx.x, head = blockIdx.y;
+  if (tok >= q_start[n_requests]) return;
+  const size_t at = ((size_t)tok * H + head) * splits;
+  const float* ml = part_ml + 2 * at;
+  const float sk = sink ? sink[head] * 1.4426950408889634f : -INFINITY;
+  float big = sk;
+  for (int s = 0; s < splits; ++s) big = fmaxf(big, ml[2 * s]);
+  float l = sink ? __builtin_amdgcn_exp2f(sk - big) : 0.f;
+  for (int s = 0; s < splits; ++s) l += ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - big);
+  const float inv = 1.0f / l;
+  const float* po = part_o + at * C;
+  for (int i = threadIdx.x * 4; i < C; i += 128 * 4) {
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < splits; ++s)
+      acc += *reinterpret_cast<const f32x4*>(po + (size_t)s * C + i) * __builtin_amdgcn_exp2f(ml[2 * s] - big);
+    bf16x4 w;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) w[e] = (__bf16)(acc[e] * inv);
+    *reinterpret_cast<bf16x4*>(out + (size_t)tok * out_tok + (size_t)head * out_head + i) = w;
   }
 }
 
@@ -482,21 +529,24 @@ latent_attention_mfma_shared_kernel(const bf16* __restrict__ q, size_t q_tok, si
 }  // namespace
 
 extern "C" int ms_latent_attention_mfma_supported(int C, int R, int page_size) {
-  return (C == 128 || C == 256 || C == 512) && (R == 32 || R == 64) && page_size > 0 && page_size % 16 == 0;
+  return (C == 64 || C == 128 || C == 192 || C == 256 || C == 384 || C == 512) && (R == 32 || R == 64) && page_size > 0 && page_size % 16 == 0;
 }
 
 // q [n, heads, C + R] (strides in elements, 16-byte aligned rows), c_pages [P, 1, page, C], r_pages [P, 1, page, R],
 // ct_pages [P, 1, C, page] (the latents once more, transposed), out [n, heads, C].  Request r owns tokens
 // q_start[r]..q_start[r+1]-1 and holds context_lens[r] keys once this step's are stored; max_q_len bounds its tokens.
+// splits > 1 (max_q_len 1 only): a tile's keys over so many blocks; part_o float [n, heads, splits, C] and part_ml float
+// [n, heads, splits, 2] for n_tokens tokens take their parts.
 extern "C" int ms_latent_attention_mfma(const void* q, long long q_tok, long long q_head, const void* c_pages,
                                         const void* r_pages, const void* ct_pages, const int* block_table,
                                         int table_stride, const int* table_rows, const int* q_start,
                                         const int* context_lens, const float* sink, void* out, long long out_tok,
                                         long long out_head, int n_requests, int max_q_len, int heads, int C, int R,
-                                        int page_size, long long num_pages, float scale, int window,
-                                        hipStream_t stream) {
+                                        int page_size, long long num_pages, float scale, int window, int splits,
+                                        int n_tokens, float* part_o, float* part_ml, hipStream_t stream) {
   if (n_requests <= 0 || max_q_len <= 0) return MS_OK;
-  if (heads <= 0 || table_stride <= 0) return MS_BAD_ARG;
+  if (heads <= 0 || table_stride <= 0 || splits <= 0) return MS_BAD_ARG;
+  if (splits > 1 && (max_q_len != 1 || !part_o || !part_ml || n_tokens <= 0 || splits > 1024)) return MS_BAD_ARG;
   if (!ms_latent_attention_mfma_supported(C, R, page_size)) return MS_UNSUPPORTED;
   if (q_tok % 8 || q_head % 8 || out_tok % 4 || out_head % 4) return MS_UNSUPPORTED;
   if (num_pages * page_size >= (1ll << 31) || n_requests > 65535) return MS_UNSUPPORTED;
@@ -505,8 +555,8 @@ extern "C" int ms_latent_attention_mfma(const void* q, long long q_tok, long lon
   // long portions: four neighbouring tiles a block over key blocks staged in LDS (more than the 64 KB a launch may
   // ask for without more ado, so the kernel's limit is raised once); else a tile's keys over the four waves
   const size_t shared_lds = ((size_t)32 * (C + R + LS_KPAD) + (size_t)C * LS_VROW) * sizeof(bf16);
-  const bool shared = tiles >= 8;
-  dim3 grid((unsigned)(shared ? (tiles + LM_WAVES - 1) / LM_WAVES : tiles), n_requests), block(LM_WAVES * MS_WAVE);
+  const bool shared = tiles >= 8 && splits == 1;
+  dim3 grid((unsigned)(shared ? (tiles + LM_WAVES - 1) / LM_WAVES : tiles), n_requests, splits), block(LM_WAVES * MS_WAVE);
 #define ARGS                                                                                                            \
       (const bf16*)q, (size_t)q_tok, (size_t)q_head, (const bf16*)c_pages, (const bf16*)r_pages, (const bf16*)ct_pages, \
       block_table, table_stride, table_rows, q_start, context_lens, sink, (bf16*)out, (size_t)out_tok,                  \
@@ -522,17 +572,27 @@ extern "C" int ms_latent_attention_mfma(const void* q, long long q_tok, long lon
         raised = true;                                                                                                  \
       }                                                                                                                 \
       latent_attention_mfma_shared_kernel<CC, RR><<<grid, block, shared_lds, stream>>>(ARGS);                           \
+    } else if (splits > 1) {                                                                                            \
+      latent_attention_mfma_kernel<CC, RR, true><<<grid, block, 0, stream>>>(ARGS, part_o, part_ml);                    \
     } else {                                                                                                            \
-      latent_attention_mfma_kernel<CC, RR><<<grid, block, 0, stream>>>(ARGS);                                           \
+      latent_attention_mfma_kernel<CC, RR, false><<<grid, block, 0, stream>>>(ARGS, nullptr, nullptr);                  \
     }                                                                                                                   \
   } while (0)
-  if (C == 128 && R == 32) LAUNCH(128, 32);
-  else if (C == 128 && R == 64) LAUNCH(128, 64);
-  else if (C == 256 && R == 32) LAUNCH(256, 32);
-  else if (C == 256 && R == 64) LAUNCH(256, 64);
-  else if (C == 512 && R == 32) LAUNCH(512, 32);
-  else LAUNCH(512, 64);
+#define SIZES(CC)                          \
+  case CC:                                 \
+    if (R == 32) LAUNCH(CC, 32);           \
+    else LAUNCH(CC, 64);                   \
+    break
+  switch (C) {
+    SIZES(64); SIZES(128); SIZES(192); SIZES(256); SIZES(384); SIZES(512);
+  }
+#undef SIZES
 #undef LAUNCH
 #undef ARGS
+  if (splits > 1) {
+    dim3 cgrid(n_tokens, heads);
+    latent_combine_kernel<<<cgrid, dim3(128), 0, stream>>>(part_o, part_ml, q_start, n_requests, sink, (bf16*)out,
+                                                           (size_t)out_tok, (size_t)out_head, heads, C, splits);
+  }
   return ms_launch_status();
 }

@@ -38,7 +38,7 @@ def memory_beside_the_pages(config: EngineConfig, model: Model, layout: CacheLay
                 size *= s
             total += (config.max_seqs + 1) * size * (n.dtype or model.rt.dtype).itemsize
     total += len(layout.group_keys) * (config.max_seqs + 1) * config.pages_per_request * 4
-    widest = max([model.spec.hidden_size * 4] + [s.shape[0] * itemsize for s in model.tensor_specs()
+    widest = max([model.spec.hidden_size * 4 * (getattr(model.embedding, "streams", None) or 1)] + [s.shape[0] * itemsize for s in model.tensor_specs()
                                                   if s.role == "matrix" and len(s.shape) == 2
                                                   and s.shape[0] != model.spec.vocab_size])
     tokens = config.max_num_batched_tokens

@@ -20,7 +20,7 @@ _CODES = {1: "bad argument", 2: "unsupported size", 3: "launch failed"}
 _c_int, _c_ll, _c_float, _c_ptr = ctypes.c_int, ctypes.c_longlong, ctypes.c_float, ctypes.c_void_p
 
 _SIGNATURES = {
-    "ms_embed": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
+    "ms_embed": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr],
     "ms_rms_norm": [_c_ptr, _c_ptr, _c_int, _c_int, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int,
                     _c_int, _c_ptr],
     "ms_rms_norm_pair": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_ptr],
@@ -91,15 +91,16 @@ _SIGNATURES = {
     "ms_concat_rows": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "ms_xielu": [_c_ptr, _c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr],
     "ms_head_matmul": [_c_ptr, _c_ll, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_ll, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int,
-                       _c_int, _c_int, _c_ptr],
+                       _c_int, _c_int, _c_int, _c_ptr],
+    "ms_head_matmul_mfma": [_c_ptr, _c_ll, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_ll, _c_ptr, _c_ll, _c_int, _c_int, _c_int,
+                            _c_int, _c_int, _c_ptr],
     "ms_rms_norm_rows": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_float, _c_int, _c_ptr],
-    "ms_rotary_pairs": [_c_ptr, _c_ll, _c_ll, _c_ptr, _c_ll, _c_ll, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int,
-                        _c_ptr],
-    "ms_latent_kv_store": [_c_ptr, _c_ll, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
-                           _c_int, _c_int, _c_int, _c_int, _c_ptr],
+    "ms_latent_prepare": [_c_ptr, _c_ll, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
+                          _c_int, _c_ptr, _c_ll, _c_ll, _c_ptr, _c_ll, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
+                          _c_ptr],
     "ms_latent_attention_mfma": [_c_ptr, _c_ll, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
                                  _c_ptr, _c_ll, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ll, _c_float,
-                                 _c_int, _c_ptr],
+                                 _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
     "ms_latent_attention": [_c_ptr, _c_ll, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
                             _c_ptr, _c_ll, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ll, _c_float, _c_int, _c_int,
                             _c_ptr],
@@ -111,7 +112,11 @@ _SIGNATURES = {
     "ms_selective_scan": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr,
                           _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "ms_gelu": [_c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr],
-    "ms_moe_route": [_c_ptr, _c_ll, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr],
+    "ms_relu2": [_c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr],
+    "ms_streams_max": [],
+    "ms_streams": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float,
+                   _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+    "ms_moe_route": [_c_ptr, _c_ll, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "ms_layer_norm": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr],
     "ms_side_gate": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "ms_mingru_chunk": [],
@@ -127,7 +132,7 @@ _SIGNATURES = {
     "ms_pooled_attention_mfma": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr,
                                  _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
                                  _c_int, _c_int, _c_ptr],
-    "ms_clamped_glu": [_c_ptr, _c_ll, _c_ptr, _c_ll, _c_int, _c_int, _c_float, _c_float, _c_int, _c_ptr],
+    "ms_clamped_glu": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_float, _c_float, _c_int, _c_ptr],
     "ms_scaled_swiglu": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_ptr],
     "ms_moe_tile_rows": [],
     "ms_moe_wide_tile_rows": [],
@@ -227,13 +232,15 @@ def _ptr(t: Optional[torch.Tensor]):
 
 # ------------------------------------------------------------------------------------------------
 def embed(ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
-    """out[n] = float(table[ids[n]]) * scale.  ids int32 [N] (checked against the table by the caller), out float32 [N, H]."""
+    """out[n] = float(table[ids[n]]) * scale.  ids int32 [N] (checked against the table by the caller), out float32 [N, H],
+    or [N, S, H]: the same row S times."""
     _check(ids, "ids", torch.int32)
     _check(table, "table")
     V, H = table.shape
-    _check(out, "out", torch.float32, (ids.numel(), H))
-    _call("ms_embed", ids.data_ptr(), table.data_ptr(), out.data_ptr(), ids.numel(), H, float(scale), _code(table.dtype),
-          _stream())
+    copies = out.shape[1] if out.dim() == 3 else 1
+    _check(out, "out", torch.float32, (ids.numel(), copies, H) if out.dim() == 3 else (ids.numel(), H))
+    _call("ms_embed", ids.data_ptr(), table.data_ptr(), out.data_ptr(), ids.numel(), H, copies, float(scale),
+          _code(table.dtype), _stream())
     return out
 
 
@@ -1168,20 +1175,37 @@ def _heads3d(t: torch.Tensor, name: str, dtype=None):
     return t.stride(0), t.stride(1)
 
 
-def head_matmul(x: torch.Tensor, m: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
+def head_maps_transposed(dtype: torch.dtype, I: int, *strides: int) -> bool:
+    """Whether ``head_matmul`` takes this type, inner size and the operand's strides (tokens, heads) to the matrix cores,
+    which read the maps as [H, J, I]."""
+    return dtype == torch.bfloat16 and I % 32 == 0 and all(st % 8 == 0 for st in strides)
+
+
+def head_matmul(x: torch.Tensor, m: torch.Tensor, out: torch.Tensor, gate: Optional[torch.Tensor] = None,
+                transposed: bool = False) -> torch.Tensor:
     """out[n, h, :] = x[n, h, :] @ m[h] (* sigmoid(gate[n, h, :])).  x [N, H, I] and out [N, H, J] may be views with any
-    token and head strides; m [H, I, J] contiguous; gate [N, H * J] rows."""
+    token and head strides; m [H, I, J] contiguous; gate rows of H * J numbers, or of H (one a head).  ``transposed``: m is
+    [H, J, I] and the product runs on the matrix cores (sizes that ``head_maps_transposed`` says)."""
     N, H, I = x.shape
     xt, xh = _heads3d(x, "x")
-    _check(m, "m", x.dtype, (H, I, None))
-    J = m.shape[2]
+    _check(m, "m", x.dtype, (H, None, I) if transposed else (H, I, None))
+    J = m.shape[1] if transposed else m.shape[2]
     ot, oh = _heads3d(out, "out")
     if tuple(out.shape) != (N, H, J):
         raise ValueError(f"out must be {[N, H, J]}, got {list(out.shape)}")
-    gs = 0
+    gs, gw = 0, J
     if gate is not None:
-        gs = _rows2d(gate, "gate", x.dtype, H * J)
-    _call("ms_head_matmul", x.data_ptr(), xt, xh, m.data_ptr(), out.data_ptr(), ot, oh, _ptr(gate), gs, N, H, I, J,
+        gw = 1 if gate.shape[1] == H else J
+        gs = _rows2d(gate, "gate", x.dtype, H * gw)
+        if gate.shape[0] != N:
+            raise ValueError("gate must have a row per token")
+    if transposed:
+        if x.dtype != torch.bfloat16 or out.dtype != torch.bfloat16:
+            raise TypeError("transposed maps are for bfloat16 in and out")
+        _call("ms_head_matmul_mfma", x.data_ptr(), xt, xh, m.data_ptr(), out.data_ptr(), ot, oh, _ptr(gate), gs, gw, N, H, I,
+              J, _stream())
+        return out
+    _call("ms_head_matmul", x.data_ptr(), xt, xh, m.data_ptr(), out.data_ptr(), ot, oh, _ptr(gate), gs, gw, N, H, I, J,
           _code(x.dtype), _code(out.dtype), _stream())
     return out
 
@@ -1197,21 +1221,12 @@ def rms_norm_rows(x: torch.Tensor, weight: torch.Tensor, eps: float, out: torch.
     return out
 
 
-def rotary_pairs(src: torch.Tensor, dst: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor) -> torch.Tensor:
-    """dst[n, h] = src[n, h] with its first 2 * len(inv_freq) entries turned, entry 2i with entry 2i + 1, by
-    float(positions[n]) * inv_freq[i]; the rest is copied.  src, dst [N, H, width] views (dst may be src)."""
-    N, H, width = src.shape
-    st, sh = _heads3d(src, "src")
-    dt, dh = _heads3d(dst, "dst", src.dtype)
-    if tuple(dst.shape) != (N, H, width):
-        raise ValueError("dst must have src's shape")
-    _check(positions, "positions", torch.int32, (N,))
-    _check(inv_freq, "inv_freq", torch.float32)
-    dims = 2 * inv_freq.numel()
-    if dims > width:
-        raise ValueError(f"{dims} rotated entries do not fit a width of {width}")
-    _call("ms_rotary_pairs", src.data_ptr(), st, sh, dst.data_ptr(), dt, dh, positions.data_ptr(), inv_freq.data_ptr(), N, H,
-          width, dims, _code(src.dtype), _stream())
+def rotary_pairs(src: torch.Tensor, dst: torch.Tensor, positions: torch.Tensor, inv_freq: torch.Tensor, gain: float = 1.0,
+                 half: bool = False) -> torch.Tensor:
+    """dst[n, h] = src[n, h] with its first 2 * len(inv_freq) entries turned, entry 2i with entry 2i + 1 (``half``: entry i
+    with entry i + len(inv_freq)), by float(positions[n]) * inv_freq[i] and multiplied by ``gain``; the rest is copied.
+    src, dst [N, H, width] views (dst may be src)."""
+    latent_prepare(positions, inv_freq, gain, half, q=(src, dst))
     return dst
 
 
@@ -1221,30 +1236,77 @@ launches = {}     # how often a dispatcher below chose a kernel that tests want 
 def latent_mfma_sizes(C: int, R: int) -> bool:
     """Whether the matrix-core attention over latents has a variant for a latent of C and a rotated part of R entries
     (the library's ms_latent_attention_mfma_supported says the same, and more about pages)."""
-    return C in (128, 256, 512) and R in (32, 64)
+    return C in (64, 128, 192, 256, 384, 512) and R in (32, 64)
+
+
+def latent_prepare(positions: torch.Tensor, inv_freq: torch.Tensor, gain: float = 1.0, half: bool = False, kv=None, q=None) -> None:
+    """What stands between latent attention's projections and the attention, one launch.  ``kv`` (rows [N, C + R],
+    norm_weight, eps, slot_mapping, c_pages, r_pages, ct_pages or None): the RMS norm of the rows' first C columns (times
+    ``norm_weight``) goes to ``c_pages`` [P, 1, page, C], their last R columns, turned, to ``r_pages`` [P, 1, page, R], at
+    ``slot_mapping`` (< 0: not stored); ``ct_pages`` [P, 1, C, page], if given, takes the same latents transposed.  ``q``
+    (src, dst), [N, heads, R] views of one type: every head's slice, turned.  Turning: ``rotary_pairs``."""
+    N = positions.numel()
+    _check(positions, "positions", torch.int32, (N,))
+    _check(inv_freq, "inv_freq", torch.float32)
+    dims = 2 * inv_freq.numel()
+    if kv is None and q is None:
+        raise ValueError("nothing to prepare")
+    store = (None, 0, None, 0.0)
+    pages = (None, None, None, None, 0)
+    query = (None, 0, 0, None, 0, 0)
+    C = R = heads = 0
+    dtype = None
+    if kv is not None:
+        rows, norm_weight, eps, slot_mapping, c_pages, r_pages, ct_pages = kv
+        dtype = rows.dtype
+        _check(c_pages, "c_pages", dtype, (None, 1, None, None))
+        C = c_pages.shape[3]
+        _check(r_pages, "r_pages", dtype, (c_pages.shape[0], 1, c_pages.shape[2], None))
+        R = r_pages.shape[3]
+        if ct_pages is not None:
+            _check(ct_pages, "ct_pages", dtype, (c_pages.shape[0], 1, C, c_pages.shape[2]))
+        ks = _rows2d(rows, "kv", None, C + R)
+        if rows.shape[0] != N:
+            raise ValueError("kv has a row per token")
+        _check(norm_weight, "norm_weight", torch.float32, (C,))
+        _check(slot_mapping, "slot_mapping", torch.int32, (N,))
+        store = (rows.data_ptr(), ks, norm_weight.data_ptr(), float(eps))
+        pages = (slot_mapping.data_ptr(), c_pages.data_ptr(), r_pages.data_ptr(), _ptr(ct_pages), c_pages.shape[2])
+    if q is not None:
+        src, dst = q
+        st, sh = _heads3d(src, "src")
+        dt, dh = _heads3d(dst, "dst", src.dtype)
+        if tuple(dst.shape) != tuple(src.shape) or src.shape[0] != N:
+            raise ValueError("dst must have src's shape, a row per token")
+        if kv is not None and (src.shape[2] != R or src.dtype != dtype):
+            raise ValueError("queries and keys have rotated parts of one size and type")
+        heads, R, dtype = src.shape[1], src.shape[2], src.dtype
+        query = (src.data_ptr(), st, sh, dst.data_ptr(), dt, dh)
+    if dims > R:
+        raise ValueError(f"{dims} rotated entries do not fit a width of {R}")
+    _call("ms_latent_prepare", *store, positions.data_ptr(), inv_freq.data_ptr(), float(gain), int(half), *pages, *query, N,
+          heads, C, R, dims, _code(dtype), _stream())
 
 
 def latent_kv_store(kv: torch.Tensor, norm_weight: torch.Tensor, eps: float, positions: torch.Tensor, inv_freq: torch.Tensor,
                     slot_mapping: torch.Tensor, c_pages: torch.Tensor, r_pages: torch.Tensor,
-                    ct_pages: Optional[torch.Tensor] = None) -> None:
-    """kv [N, C + R]: the RMS norm of its first C columns (times ``norm_weight``) goes to ``c_pages`` [P, 1, page, C], its
-    last R columns, turned pair by pair, to ``r_pages`` [P, 1, page, R], at ``slot_mapping`` (< 0: not stored).
-    ``ct_pages`` [P, 1, C, page], if given, takes the same latents transposed."""
-    N = kv.shape[0]
-    _check(c_pages, "c_pages", kv.dtype, (None, 1, None, None))
-    C = c_pages.shape[3]
-    _check(r_pages, "r_pages", kv.dtype, (c_pages.shape[0], 1, c_pages.shape[2], None))
-    R = r_pages.shape[3]
-    if ct_pages is not None:
-        _check(ct_pages, "ct_pages", kv.dtype, (c_pages.shape[0], 1, C, c_pages.shape[2]))
-    ks = _rows2d(kv, "kv", None, C + R)
-    _check(norm_weight, "norm_weight", torch.float32, (C,))
-    _check(positions, "positions", torch.int32, (N,))
-    _check(slot_mapping, "slot_mapping", torch.int32, (N,))
-    _check(inv_freq, "inv_freq", torch.float32)
-    _call("ms_latent_kv_store", kv.data_ptr(), ks, norm_weight.data_ptr(), float(eps), positions.data_ptr(),
-          inv_freq.data_ptr(), slot_mapping.data_ptr(), c_pages.data_ptr(), r_pages.data_ptr(), _ptr(ct_pages),
-          c_pages.shape[2], N, C, R, 2 * inv_freq.numel(), _code(kv.dtype), _stream())
+                    ct_pages: Optional[torch.Tensor] = None, gain: float = 1.0, half: bool = False) -> None:
+    """``latent_prepare`` without queries."""
+    latent_prepare(positions, inv_freq, gain, half, kv=(kv, norm_weight, eps, slot_mapping, c_pages, r_pages, ct_pages))
+
+
+LATENT_SPLIT_BLOCKS = 512     # blocks a step of single tokens aims to put on the chip
+
+
+def latent_splits(n_requests: int, heads: int, max_q_len: int, max_context_len: int, window: Optional[int]) -> int:
+    """Over how many blocks the matrix-core attention over latents spreads a tile's keys: a launch constant of the batch
+    size and of the longest context the step is made for.  A block's four waves take four key blocks of 32 at a time."""
+    if max_q_len != 1:
+        return 1
+    keys = min(max_context_len, window + 31) if window else max_context_len
+    tiles = n_requests * -(-heads // 16)
+    most = 16 if keys <= 16384 else (32 if keys <= 65536 else 128)
+    return max(1, min(most, LATENT_SPLIT_BLOCKS // max(1, tiles), -(-keys // 128)))
 
 
 def latent_attention(q: torch.Tensor, kv, ctx, out: torch.Tensor, scale: float, window: Optional[int] = None,
@@ -1281,10 +1343,16 @@ def latent_attention(q: torch.Tensor, kv, ctx, out: torch.Tensor, scale: float, 
         Rq = ctx.num_requests
         _check(ctx.q_start, "q_start", torch.int32, (Rq + 1,))
         _check(ctx.context_lens, "context_lens", torch.int32, (Rq,))
+        splits = latent_splits(Rq, H, ctx.max_q_len, int(getattr(ctx, "max_context_len", 0)), window)
+        part_o = part_ml = None
+        if splits > 1:
+            launches["latent_attention_split"] = launches.get("latent_attention_split", 0) + 1
+            part_o = torch.empty((N, H, splits, C), dtype=torch.float32, device=q.device)
+            part_ml = torch.empty((N, H, splits, 2), dtype=torch.float32, device=q.device)
         _call("ms_latent_attention_mfma", q.data_ptr(), qt, qh, c_pages.data_ptr(), r_pages.data_ptr(), ct_pages.data_ptr(),
               kv.block_table.data_ptr(), kv.block_table.shape[1], _ptr(kv.table_rows), ctx.q_start.data_ptr(),
               ctx.context_lens.data_ptr(), _ptr(sink), out.data_ptr(), ot, oh, Rq, ctx.max_q_len, H, C, R, page_size, P,
-              float(scale), int(window or 0), _stream())
+              float(scale), int(window or 0), splits, N, _ptr(part_o), _ptr(part_ml), _stream())
         return out
     _call("ms_latent_attention", q.data_ptr(), qt, qh, c_pages.data_ptr(), r_pages.data_ptr(), kv.block_table.data_ptr(),
           kv.block_table.shape[1], _ptr(kv.table_rows), _ptr(ctx.n_live_tokens), ctx.token_req.data_ptr(),
@@ -1416,11 +1484,21 @@ def gelu(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
     return out
 
 
+def relu2(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out = max(x, 0)^2."""
+    _check(x, "x")
+    _check(out, "out", x.dtype, tuple(x.shape))
+    _call("ms_relu2", x.data_ptr(), out.data_ptr(), x.numel(), _code(x.dtype), _stream())
+    return out
+
+
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, n_out: Optional[int] = None,
-              scores: str = "softmax"):
+              scores: str = "softmax", groups=None, normalise: bool = False):
     """Scores = softmax(logits[:, :n_out]) (``scores`` "sigmoid": every logit's own sigmoid); the ``top`` largest of
     scores + correction are chosen (the lower index on a tie).  Returns (ids int32 [N, top], their scores float [N, top]).
-    logits float [N, >= n_out]."""
+    logits float [N, >= n_out].  ``groups`` (count, keep): the outputs form ``count`` equal groups of neighbours, a group
+    counts as its largest score + correction, and only outputs of the ``keep`` best groups can be chosen.  ``normalise``:
+    the chosen scores are divided by (their sum + 1e-20)."""
     if scores not in ("softmax", "sigmoid"):
         raise ValueError(f"router scores are 'softmax' or 'sigmoid', not {scores!r}")
     ld = _rows2d(logits, "logits", torch.float32)
@@ -1430,10 +1508,13 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
         raise ValueError(f"top {top} of {n_out} outputs in rows of {logits.shape[1]}")
     if correction is not None:
         _check(correction, "correction", torch.float32, (n_out,))
+    count, keep = groups if groups is not None else (0, 0)
+    if groups is not None and (count <= 0 or n_out % count or not 0 < keep <= count or top > keep * (n_out // count)):
+        raise ValueError(f"top {top} of {n_out} outputs within {keep} of {count} equal groups")
     ids = torch.empty((N, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((N, top), dtype=torch.float32, device=logits.device)
     _call("ms_moe_route", logits.data_ptr(), ld, _ptr(correction), N, n_out, top, ids.data_ptr(), weights.data_ptr(),
-          int(scores == "sigmoid"), _stream())
+          int(scores == "sigmoid"), count, keep, int(normalise), _stream())
     return ids, weights
 
 
@@ -1516,8 +1597,8 @@ def grouped_gemm(a: torch.Tensor, w: torch.Tensor, rows: torch.Tensor, tile_expe
 
 def moe_combine(part: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, h: torch.Tensor, n_experts: int,
                 out: torch.Tensor, shared: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """out[n] = sum_j weights[n, j] * (part[n * top + j] if ids[n, j] < n_experts else h[n]) + sigmoid(gate[n]) * shared[n].
-    part float [N * top, H]; h [N, H]; shared [N, H] (h's type or float) with gate float [N] (a column of a wider matrix
+    """out[n] = sum_j weights[n, j] * (part[n * top + j] if ids[n, j] < n_experts else h[n]) + sigmoid(gate[n]) * shared[n]
+    (``gate`` None: + shared[n]).  part float [N * top, H]; h [N, H]; shared [N, H] (h's type or float) with gate float [N] (a column of a wider matrix
     is fine); out float [N, H]."""
     N, top = ids.shape
     _check(ids, "ids", torch.int32)
@@ -1531,10 +1612,11 @@ def moe_combine(part: torch.Tensor, ids: torch.Tensor, weights: torch.Tensor, h:
     if shared is not None:
         _check(shared, "shared", None, (N, H))
         scode = _code(shared.dtype)
-        _check(gate, "gate", torch.float32, contiguous=False)
-        if gate.dim() != 1 or gate.shape[0] != N:
-            raise ValueError("gate must be one float per token")
-        gs = gate.stride(0) if N > 1 else 1
+        if gate is not None:
+            _check(gate, "gate", torch.float32, contiguous=False)
+            if gate.dim() != 1 or gate.shape[0] != N:
+                raise ValueError("gate must be one float per token")
+            gs = gate.stride(0) if N > 1 else 1
     _call("ms_moe_combine", part.data_ptr(), ids.data_ptr(), _ptr(weights), h.data_ptr(), hs, _ptr(shared), scode,
           _ptr(gate), gs, out.data_ptr(), N, top, n_experts, H, _code(h.dtype), _stream())
     return out
@@ -1741,16 +1823,77 @@ def pooled_attention(q: torch.Tensor, kv, pooled, ctx, out: torch.Tensor, num_he
     return out
 
 
+# ------------------------------------------------------------------------------------------------ several residual streams
+NORM_KINDS = {None: 0, "rms": 1, "layer": 2}
+
+
+STREAMS_MAX = 32     # the library's ms_streams_max()
+
+
+def streams_step(x: torch.Tensor, write=None, read=None, rows: Optional[torch.Tensor] = None, write_back: bool = True):
+    """A residual stream made of S copies, x float [N, S, W]; one pass.
+    ``write`` (y, mix [S, S], b [S]): x[t] <- sum_s mix[s, t] x[s] + b[t] y, all t from the old x.  y: a tensor [N, W], or
+    (base [N, W] or None, part float [N * top, W], weights float [N, top]) for base[n] + sum_j weights[n, j] part[n top + j].
+    ``read`` (a [S], kind, weight, bias, eps, out [n, W]): out = norm(sum_s a[s] x[s]) of the new x, kind None, "rms" or
+    "layer".  ``rows`` int32: only those rows; ``write_back`` False: the written streams are read but not kept."""
+    _check(x, "x", torch.float32)
+    if x.dim() != 3:
+        raise ValueError(f"the streams are [tokens, streams, width], got {list(x.shape)}")
+    N, S, W = x.shape
+    n_rows = N
+    if rows is not None:
+        _check(rows, "rows", torch.int32)
+        n_rows = rows.numel()
+        if write is not None and write_back:
+            raise ValueError("chosen rows are read only (write_back=False)")
+    base = part = weights = mix = b = None
+    base_code, top = F32, 0
+    if write is not None:
+        y, mix, b = write
+        if isinstance(y, tuple):
+            base, part, weights = y
+            top = weights.shape[1]
+            _check(weights, "weights", torch.float32, (N, top))
+            _check(part, "part", torch.float32, (N * top, W))
+        else:
+            base = y
+        if base is not None:
+            _check(base, "y", None, (N, W))
+            base_code = _code(base.dtype)
+        _check(mix, "mix", torch.float32, (S, S))
+        _check(b, "b", torch.float32, (S,))
+    a = weight = bias = out = None
+    kind, eps, out_code = 0, 0.0, F32
+    if read is not None:
+        a, name, weight, bias, eps, out = read
+        kind = NORM_KINDS[name]
+        _check(a, "a", torch.float32, (S,))
+        if kind:
+            _check(weight, "weight", torch.float32, (W,))
+        if bias is not None:
+            _check(bias, "bias", torch.float32, (W,))
+        _check(out, "out", None, (n_rows, W))
+        out_code = _code(out.dtype)
+    _call("ms_streams", x.data_ptr(), _ptr(base), base_code, _ptr(part), _ptr(weights), top, _ptr(mix), _ptr(b), _ptr(a), kind,
+          _ptr(weight), _ptr(bias), float(eps), _ptr(rows), _ptr(out), out_code, n_rows, S, W, int(write_back), _stream())
+    return out
+
+
 # ------------------------------------------------------------------------------------------------ gated activations
-def clamped_glu(gu: torch.Tensor, out: torch.Tensor, limit: float, alpha: float = 1.702) -> torch.Tensor:
+def clamped_glu(gu: torch.Tensor, out: torch.Tensor, limit: float, alpha: float = 1.702,
+                row_item: Optional[torch.Tensor] = None) -> torch.Tensor:
     """gu [N, 2F] with gate and up interleaved: g = min(g, limit), u = clamp(u, -limit, limit),
-    out = g * sigmoid(alpha g) * (u + 1), [N, F]."""
+    out = g * sigmoid(alpha g) * (u + 1), [N, F].  Rows with a negative ``row_item`` are left alone."""
     F = gu.shape[1] // 2
     s_in = _rows2d(gu, "gu", None, 2 * F)
     s_out = _rows2d(out, "out", gu.dtype, F)
     if out.shape[0] != gu.shape[0]:
         raise ValueError("out has one row per row of gu")
-    _call("ms_clamped_glu", gu.data_ptr(), s_in, out.data_ptr(), s_out, gu.shape[0], F, float(limit), float(alpha),
+    if row_item is not None:
+        _check(row_item, "row_item", torch.int32)
+        if row_item.numel() < gu.shape[0]:
+            raise ValueError("row_item names an item for every row")
+    _call("ms_clamped_glu", gu.data_ptr(), s_in, _ptr(row_item), out.data_ptr(), s_out, gu.shape[0], F, float(limit), float(alpha),
           _code(gu.dtype), _stream())
     return out
 

@@ -3,7 +3,8 @@
 A part is built from the sizes and constants in its ``PartSpec`` alone and never learns which model
 it is in.  Five kinds are chosen layer by layer:
 
-``Norm``              forward(x, delta, rows, write_back) -> activations         (x: the float residual stream)
+``Norm``              forward(x, delta, rows, write_back) -> activations         (x: the float residual stream; ``statistic``:
+                      what it divides by, for kernels that take the norm on their way)
 ``PositionEncoding``  encode_and_store(qkv, nh, nkv, d, ctx, kv)                 (belongs to a mixer)
 ``Mixer``             forward(h, ctx, kv, state) -> [N, hidden]                  (attention here)
 ``FeedForward``       forward(h, ctx) -> [N, hidden]
@@ -205,6 +206,10 @@ class Part:
 
 
 class Norm(Part):
+    # "rms" (x over its root mean square) or "layer" (mean taken off first): the norm is that, times ``weight``, plus
+    # ``bias`` (None: none), with ``eps``, and a kernel that has the row at hand may take it itself.  None: only ``forward``.
+    statistic: Optional[str] = None
+
     def lazy(self, x: torch.Tensor, delta: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None,
              write_back: bool = True):
         """What a block calls for a consumer that declares ``accepts_lazy_norm``: may return an object that
@@ -282,6 +287,11 @@ class FeedForward(Part):
 
     def forward_residual(self, h: torch.Tensor, ctx: StepContext, x: torch.Tensor) -> Optional[torch.Tensor]:
         """As ``Mixer.forward_residual``."""
+        return self.forward(h, ctx)
+
+    def forward_deferred(self, h: torch.Tensor, ctx: StepContext):
+        """For a block whose next kernel can do the last sum itself: ``forward``'s result, or (base [N, hidden] or None,
+        rows float [N * k, hidden], weights float [N, k]) for base[n] + sum_j weights[n, j] rows[n k + j]."""
         return self.forward(h, ctx)
 
 
@@ -465,7 +475,7 @@ class Head(Part):
 # ------------------------------------------------------------------------------------------------ registries
 _REGISTRIES: Dict[str, Dict[str, type]] = {
     "norm": {}, "position": {}, "mixer": {}, "feed_forward": {}, "filter": {}, "block": {}, "embedding": {}, "head": {},
-    "pass_entry": {}, "scale": {}, "token_input": {},
+    "pass_entry": {}, "scale": {}, "token_input": {}, "stream_link": {},
 }
 
 

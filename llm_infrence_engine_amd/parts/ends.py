@@ -3,6 +3,8 @@ src/miniserve/model.py:229) and the output head (a matrix product with the head'
 tied, the embedding table, model.py:204-206, 237).  Logits are float."""
 from __future__ import annotations
 
+from typing import Optional
+
 import torch
 
 from ..kernels import linear, ops
@@ -11,12 +13,17 @@ from .base import Embedding, Head, PassEntry, build_part, register_part
 
 
 class TokenEmbedding(Embedding):
-    def __init__(self, prefix: str, vocab_size: int, hidden_size: int, name: str = "weight", scale: float = 1.0, norm=None):
+    def __init__(self, prefix: str, vocab_size: int, hidden_size: int, name: str = "weight", scale: float = 1.0, norm=None,
+                 streams: Optional[int] = None):
         """``scale``: every row is multiplied by it on its way into the float residual stream.  ``norm``: the
-        ``PartSpec`` of a norm that the rows pass right after (one with ``normalize_``), or None."""
+        ``PartSpec`` of a norm that the rows pass right after (one with ``normalize_``), or None.  ``streams``: the residual
+        stream has so many copies, [N, streams, hidden_size], all equal here (None: it is [N, hidden_size])."""
         self.prefix, self.vocab_size, self.hidden_size, self.name = prefix, vocab_size, hidden_size, name
         self.scale = float(scale)
         self.norm = build_part("norm", norm) if norm is not None else None
+        self.streams = streams
+        if streams is not None and (streams <= 0 or norm is not None):
+            raise ValueError("streams come in a positive number, and without a norm of the embedding's rows")
         if self.norm is not None and not hasattr(self.norm, "normalize_"):
             raise ValueError(f"the norm {norm.kind!r} cannot be applied in place to the embedding's rows")
 
@@ -31,7 +38,8 @@ class TokenEmbedding(Embedding):
             self.norm.load(get, rt)
 
     def forward(self, ctx):
-        out = self.rt.empty(ctx.num_tokens, self.hidden_size, dtype=torch.float32)
+        copies = () if self.streams is None else (self.streams,)
+        out = self.rt.empty(ctx.num_tokens, *copies, self.hidden_size, dtype=torch.float32)
         ops.embed(ctx.token_ids, self.weight, out, self.scale)
         return self.norm.normalize_(out) if self.norm is not None else out
 

@@ -37,9 +37,9 @@ class SwiGLU(FeedForward):
 class DenseAct(FeedForward):
     """down(act(up(x))), no biases.  ``activation``: "xielu", with two learned numbers (p, q) in the tensor ``act``:
     z > 0: softplus(p) z^2 + z/2;  z <= 0: (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2; or "gelu", the exact one,
-    z/2 (1 + erf(z / sqrt 2)), which has no tensor."""
+    z/2 (1 + erf(z / sqrt 2)), or "relu2", max(z, 0)^2; these have no tensor."""
 
-    ACTIVATIONS = ("xielu", "gelu")
+    ACTIVATIONS = ("xielu", "gelu", "relu2")
 
     def __init__(self, prefix: str, hidden_size: int, intermediate_size: int, activation: str = "xielu"):
         if activation not in self.ACTIVATIONS:
@@ -61,7 +61,10 @@ class DenseAct(FeedForward):
 
     def forward_residual(self, h, ctx, x):
         u = linear.linear(h, self.w_up)
-        u = ops.xielu(u, self.act, torch.empty_like(u)) if self.activation == "xielu" else ops.gelu(u, torch.empty_like(u))
+        if self.activation == "xielu":
+            u = ops.xielu(u, self.act, torch.empty_like(u))
+        else:
+            u = (ops.gelu if self.activation == "gelu" else ops.relu2)(u, torch.empty_like(u))
         return linear.linear_residual(u, self.w_down, None, x)
 
 

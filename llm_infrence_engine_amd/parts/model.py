@@ -14,7 +14,7 @@ from ..config.spec import ModelSpec
 from ..weights.reader import CheckpointReader, place
 from ..weights.spec import TensorSpec
 from . import (attention, blocks, delta, ends, experts, feed_forward, filters, latent, linear_attention, mingru,  # noqa: F401
-               norms, pooled_attention, positions, scan, side, side_by_side)      # (register the built-in parts)
+               norms, pooled_attention, positions, scan, side, side_by_side, streams)      # (register the built-in parts)
 from .base import KVView, Runtime, StateView, StepContext, build_part, part_class, weakest
 
 
@@ -91,8 +91,8 @@ class Model:
         return self.head_logits(x, pending, ctx.logit_rows)
 
     def forward_hidden(self, ctx: StepContext, caches: List[RunCache]):
-        """Embedding and all runs of the order: the float residual stream [N, H] and the last run's addend that
-        is still to be summed into it (or None)."""
+        """Embedding and all runs of the order: the float residual stream ([N, H], or [N, S, H] where the model has S
+        copies of it) and what the last run has still to write into it (an addend, a ``StreamsWrite``, or None)."""
         x = self.embedding.forward(ctx)
         kept = x.clone() if self.pass_entry is not None and self.pass_entry.keeps_embedding else None
         pending = None
@@ -101,7 +101,7 @@ class Model:
                 if pending is not None:      # the pass's addends go into the sum itself
                     from ..kernels import ops
 
-                    ops.residual_add(x, pending)
+                    pending.add_into(x) if hasattr(pending, "add_into") else ops.residual_add(x, pending)
                     pending = None
                 new = self.pass_entry.forward(x, kept, run.opens_pass)
                 x = x if new is None else new

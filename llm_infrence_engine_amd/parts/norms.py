@@ -16,6 +16,9 @@ from .base import Norm, register_part
 
 
 class RMSNorm(Norm):
+    statistic = "rms"
+    bias = None
+
     def __init__(self, prefix: str, size: int, eps: float, offset: float = 0.0, name: str = "weight", gain: float = 1.0):
         self.prefix, self.size, self.eps, self.offset, self.name = prefix, size, eps, float(offset), name
         self.gain = float(gain)
@@ -78,6 +81,7 @@ class LayerNorm(Norm):
     element, on its way into x (a layer's scale)."""
 
     takes_delta_scale = True
+    statistic = "layer"
 
     def __init__(self, prefix: str, size: int, eps: float, name: str = "weight", bias_name: str = None, gain: float = 1.0):
         self.prefix, self.size, self.eps, self.name = prefix, size, float(eps), name

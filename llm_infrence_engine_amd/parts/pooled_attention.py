@@ -34,6 +34,8 @@ class PooledWindowAttention(Mixer):
             raise ValueError("key and value sizes are even and at most 256")
         if size <= 0 or pool <= 0:
             raise ValueError("the window and the pooled blocks hold at least one token")
+        if getattr(position, "half", False) or getattr(position, "scaling", None) is not None:
+            raise ValueError("this mixer turns pairs of neighbours by unscaled frequencies")
         if position is not None and not hasattr(position, "inv_freq") and not hasattr(position, "dims"):
             raise ValueError("this mixer turns pairs of neighbours: it takes the position encoding 'rotary_pairs' or none")
         self.prefix, self.position = prefix, position

@@ -65,23 +65,29 @@ class NoPosition(PositionEncoding):
 
 
 class RotaryPairs(PositionEncoding):
-    """Rotary encoding with neighbouring entries paired: of a vector's first ``dims`` entries, entry 2i and entry
-    2i + 1 turn by position * theta^(-2i/dims); the rest pass unchanged.  It turns whatever slice of a vector its
-    mixer hands it (``rotate``); angles, sines and cosines are float."""
+    """Rotary encoding of a slice of a vector: of its first ``dims`` entries, entry 2i and entry 2i + 1 (``pairing``
+    "neighbours"), or entry i and entry i + dims / 2 ("half"), turn by position * f_i and are multiplied by ``gain``; the
+    rest pass unchanged.  f_i = theta^(-2i/dims), or with ``scaling`` (YaRN's keys) what ``yarn_frequencies`` makes of it,
+    which also gives the gain.  It turns whatever slice its mixer hands it; angles, sines and cosines are float."""
 
-    def __init__(self, prefix: str, width: int, dims: int, theta: float):
+    def __init__(self, prefix: str, width: int, dims: int, theta: float, pairing: str = "neighbours", scaling=None):
         if dims % 2 or not 0 <= dims <= width:
             raise ValueError(f"{dims} rotated entries must be even and within the vector's width {width}")
+        if pairing not in ("neighbours", "half"):
+            raise ValueError(f"entries are paired as 'neighbours' or by 'half', not {pairing!r}")
         self.width, self.dims, self.theta = width, dims, float(theta)
+        self.half = pairing == "half"
+        self.scaling = dict(scaling) if scaling is not None else None
+        self.gain = 1.0
 
     def load(self, get, rt):
         self.rt = rt
-        i = torch.arange(0, self.dims, 2, dtype=torch.float64)
-        self.inv_freq = (self.theta ** (-i / max(1, self.dims))).to(torch.float32).to(rt.device)
+        f, self.gain = yarn_frequencies(self.dims, self.theta, self.scaling)
+        self.inv_freq = f.to(torch.float32).to(rt.device)
 
     def rotate(self, src, dst, ctx):
         """dst[n, h] = src[n, h] turned by the position of token n; [N, heads, width] views, dst may be src."""
-        return ops.rotary_pairs(src, dst, ctx.positions, self.inv_freq)
+        return ops.rotary_pairs(src, dst, ctx.positions, self.inv_freq, self.gain, self.half)
 
 
 class QKNormTemperature(PositionEncoding):
@@ -121,6 +127,25 @@ class QKNormTemperature(PositionEncoding):
                           self.q_weight, self.k_weight, self.eps, ctx.positions, self.coef, self.every,
                           kv.slot_mapping if store else None, kv.k_pages if store else None,
                           kv.v_pages if store else None, bool(store and kv.v_transposed))
+
+
+def yarn_frequencies(dims: int, base: float, scaling=None):
+    """(f_i = base^(-2 i / dims) for i < dims / 2 in double, the factor of cosines and sines).  ``scaling`` {"factor",
+    "original", "fast", "slow"}: pair i keeps f_i below a ramp over the pair's index, has f_i / factor above it and a blend
+    on it; the ramp's ends are the indices, rounded outwards, of pairs that turn ``fast`` and ``slow`` times within
+    ``original`` positions; cosines and sines are multiplied by 0.1 ln(factor) + 1."""
+    i = torch.arange(0, dims // 2, dtype=torch.float64)
+    f = float(base) ** (-2.0 * i / max(1, dims))
+    if scaling is None:
+        return f, 1.0
+    factor, original, fast, slow = (float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
+
+    def index(turns):
+        return dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(float(base)))
+
+    lo, hi = max(math.floor(index(fast)), 0), min(math.ceil(index(slow)), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return f / factor * ramp + f * (1.0 - ramp), 0.1 * math.log(factor) + 1.0
 
 
 def scaled_frequencies(dims: int, base: float, scaling=None) -> torch.Tensor:

@@ -2,7 +2,7 @@
 
 The reference has no such mode (its loader only reads checkpoints, src/miniserve/loader.py:29-51).
 Tensors are drawn in the order the model's parts list them, in float on the CPU from one seeded
-generator: matrices and biases N(0, std), norm scales 1 + N(0, 0.1); then stored in ``dtype``.
+generator: matrices and biases N(0, std), norm scales 1 + N(0, 0.1), mixing matrices of stream copies the identity + N(0, std); then stored in ``dtype``.
 
 ``load_random_model`` is the same mode without the folder, for models too large to pass through host
 memory and a file: every tensor is drawn on the GPU, piece by piece, straight in the type it is kept in.
@@ -29,6 +29,8 @@ def random_tensors(specs, seed: int, std: float = 0.02, norm_std: float = 0.1, d
             continue
         t = torch.randn(s.shape, generator=g, dtype=torch.float32)
         t = 1.0 + norm_std * t if s.role == "norm" else std * t
+        if s.role == "mixing":
+            t = t + torch.eye(s.shape[0])
         out[s.name] = t.to(_STORE[dtype]).contiguous()
     return out
 
@@ -73,7 +75,7 @@ class RandomSource:
         if s.role == "table":
             return torch.zeros(s.shape, dtype=torch.int32, device=self.device)
         g = torch.Generator(device=self.device).manual_seed((self.seed * 1000003 + i) & ((1 << 62) - 1))
-        keep = torch.float32 if s.role in ("bias", "norm") or s.keep32 else self.run_dtype
+        keep = torch.float32 if s.role in ("bias", "norm", "mixing") or s.keep32 else self.run_dtype
         out = torch.empty(s.shape, dtype=keep, device=self.device)
         flat = out.view(-1)
         for a in range(0, flat.numel(), self.piece):
@@ -81,6 +83,8 @@ class RandomSource:
             t = torch.randn(b - a, generator=g, dtype=torch.float32, device=self.device)
             t = t.mul_(self.norm_std).add_(1.0) if s.role == "norm" else t.mul_(self.std)
             flat[a:b].copy_(t)
+        if s.role == "mixing":
+            out += torch.eye(s.shape[0], dtype=out.dtype, device=self.device)
         return out
 
     def close(self) -> None:

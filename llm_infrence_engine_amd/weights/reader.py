@@ -123,7 +123,7 @@ def place(t: torch.Tensor, spec: TensorSpec, run_dtype: torch.dtype, device) -> 
     stored in 32-bit float stays so when its part says ``keep32``), vectors in float, integer tables as int32."""
     if spec.role == "table":
         return t.to(device=device, dtype=torch.int32).contiguous()
-    if spec.role in ("bias", "norm"):
+    if spec.role in ("bias", "norm", "mixing"):
         return t.to(device=device, dtype=torch.float32).contiguous()
     if spec.keep32 and t.dtype == torch.float32:
         return t.to(device=device).contiguous()
