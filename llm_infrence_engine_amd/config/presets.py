@@ -1,5 +1,5 @@
 """Named config.json contents for the random-weights mode: the shapes the published Qwen2.5 checkpoints
-have, the two tiny ones the tests use and two Gemadra, two Gidurax and two Kuvazen shapes of the same widths, so that ``--random-config 0.5b``
+have, the two tiny ones the tests use and two Gemadra, two Gidurax, two Kuvazen, two Silizen and two Gositar shapes of the same widths, so that ``--random-config 0.5b``
 needs no file.  These are data
 of the kind a config.json holds; no part or kernel reads them.
 """
@@ -120,6 +120,30 @@ PRESETS["silizen-7b"] = _silizen(
     3584, 18944, 28, {"heads": 28, "kv_heads": 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5},
     {"heads": 28, "dim": 64, "vdim": 128}, {"heads": 28, "kv_heads": 14, "dim": 128, "vdim": 128}, {"heads": 28, "dim": 128}, 1024,
     128, vocab=152064)
+
+
+def _gositar(width, ff, layers, streams, latent, experts, vocab=151936):
+    """``layers`` layers, attention of the ungated kind but for every fourth one (the third), every second feed-forward routed
+    (``experts``: (expert ff, experts, top, groups, kept groups, shared ff))."""
+    import copy
+
+    ef, n, top, count, keep, shared = experts
+    routed = {"kind": "moe", "expert": {"ff": ef, "limit": 7.0}, "router": {"experts": n, "top": top,
+              "groups": {"count": count, "keep": keep}}, "shared": {"ff": shared, "limit": 7.0}}
+    return {"architecture": "Gositar", "vocab": vocab, "width": width, "streams": streams, "norm": {"eps": 1e-6},
+            "layers": [{"type": "latent_attention" if i % 4 == 2 else "latent_attention_2", "mixer": copy.deepcopy(latent),
+                        "mlp": copy.deepcopy(routed) if i % 2 else {"kind": "dense", "ff": ff}} for i in range(layers)]}
+
+
+# Gositar at the same widths: latent attention of Gemadra's sizes (over all keys), dense feed-forwards of Gemadra's size,
+# routed ones whose two chosen experts of sixteen and shared expert together have the Qwen2 shapes' gated size
+_YARN = {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}
+PRESETS["gositar-0.5b"] = _gositar(
+    896, 7296, 24, 4, {"heads": 14, "dim": 64, "rot_dim": 32, "vdim": 64, "kv_rank": 256, "scale": 96 ** -0.5,
+                       "rot": {"base": 10000.0, "dims": 32, "scaling": _YARN}}, (1600, 16, 2, 4, 2, 1664))
+PRESETS["gositar-7b"] = _gositar(
+    3584, 28416, 28, 4, {"heads": 28, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
+                         "rot": {"base": 10000.0, "dims": 64, "scaling": _YARN}}, (6336, 16, 2, 4, 2, 6272), vocab=152064)
 
 
 def preset(name: str) -> dict:

@@ -262,25 +262,34 @@ latent_combine_kernel(const float* __restrict__ part_o, const float* __restrict_
   }
 }
 
-// The shape for long portions: the four waves of a block own four neighbouring tiles (64 columns, whose key ranges
-// all but coincide) and read every key block from LDS, where the block's threads have put it together once: the
-// keys as rows of C + R entries, the transposed latents as rows of 32 keys, both padded so that the fragments'
-// reads spread over the banks.  A key block then comes from the L2 once for 64 columns instead of once for 16.
-constexpr int LS_KPAD = 8, LS_VROW = 40;     // entries: a key's row is C + R + 8 long, a latent entry's row 32 + 8
+// The shape for long portions: the WAVES waves of a block own neighbouring tiles of 16 columns, whose key ranges all but
+// coincide, and read every key block of 32 from LDS.  A key block goes from memory straight to LDS (global_load_lds, 16
+// bytes a lane, no registers) into one of two buffers, one block ahead of the one that is multiplied, and its page ids are
+// looked up one block before that; a step has one barrier.  In LDS a key is a row of C + R entries and a latent entry of the
+// transposed copy a row of the block's 32 keys, both in pieces of 16 bytes whose places are permuted by the row so that
+// fragment reads spread over the banks.  Blocks with the latest columns, which have the most keys, start first.
+template <int C, int R> struct Staged {
+  static constexpr int KP = (C + R) / 8;                                   // pieces of a key's row
+  static constexpr int SHIFT = KP % 16 == 8 ? 1 : (KP % 16 == 0 ? 0 : 2);  // neighbouring rows start 32, 0 or 16 / 48 banks apart
+  static constexpr int MASK = SHIFT == 2 ? 3 : 7;
+  static_assert(C % 64 == 0 && (R / 8) % (MASK + 1) == 0, "pieces are permuted within whole groups");
+  static constexpr int K_LOADS = 32 * KP / MS_WAVE, V_LOADS = C * 4 / MS_WAVE;    // loads of 64 pieces (1 KB)
+  static constexpr size_t BUFFER = (size_t)(K_LOADS + V_LOADS) * MS_WAVE * 8;     // entries of one buffer
+};
 
-template <int C, int R>
-__global__ void __launch_bounds__(LM_WAVES * MS_WAVE)
-latent_attention_mfma_shared_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_head,
+template <int C, int R, int WAVES>
+__global__ void __launch_bounds__(WAVES * MS_WAVE)
+latent_attention_mfma_staged_kernel(const bf16* __restrict__ q, size_t q_tok, size_t q_head,
                                     const bf16* __restrict__ c_pages, const bf16* __restrict__ r_pages,
                                     const bf16* __restrict__ ct_pages, const int* __restrict__ block_table,
                                     int table_stride, const int* __restrict__ table_rows,
                                     const int* __restrict__ q_start, const int* __restrict__ context_lens,
                                     const float* __restrict__ sink, bf16* __restrict__ out, size_t out_tok,
                                     size_t out_head, int H, int page_size, float scale_log2e, int window) {
-  constexpr int KS_C = C / 32, KS_R = R / 32, CT = C / 16, KROW = C + R + LS_KPAD;
-  extern __shared__ __align__(16) bf16 ls[];
-  bf16* Ks = ls;                       // [32][KROW]
-  bf16* Vs = ls + 32 * KROW;           // [C][LS_VROW]
+  using L = Staged<C, R>;
+  constexpr int KS_C = C / 32, KS_R = R / 32, CT = C / 16;
+  constexpr int LOADS = (L::K_LOADS + L::V_LOADS + WAVES - 1) / WAVES;
+  extern __shared__ __align__(16) bf16 ls[];       // two buffers: keys [32][C + R], then transposed latents [C][32]
   const int lane = threadIdx.x & (MS_WAVE - 1);
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / MS_WAVE);
   const int col16 = lane & 15, kq = lane >> 4;
@@ -288,18 +297,17 @@ latent_attention_mfma_shared_kernel(const bf16* __restrict__ q, size_t q_tok, si
   const int q0 = q_start[r];
   const int qlen = q_start[r + 1] - q0;
   const int ncols = qlen * H;
-  const int b0 = blockIdx.x * 16 * LM_WAVES;        // the block's first column
+  const int b0 = (int)(gridDim.x - 1 - blockIdx.x) * 16 * WAVES;        // the block's first column
   if (b0 >= ncols) return;                         // the whole block
   const int start_pos = context_lens[r] - qlen;
   const int* table = block_table + (size_t)(table_rows ? table_rows[r] : r) * table_stride;
   // the block's keys: from the first column's window to the last column's own position
-  const int blk_hi = start_pos + (min(ncols, b0 + 16 * LM_WAVES) - 1) / H;
+  const int blk_hi = start_pos + (min(ncols, b0 + 16 * WAVES) - 1) / H;
   const int blk_lo = window > 0 ? max(0, start_pos + b0 / H - window + 1) : 0;
   // this wave's tile and this lane's column
   const int c0 = b0 + wave * 16;
   const bool tile = c0 < ncols;
-  const int last_col = min(ncols, c0 + 16) - 1;
-  const int key_hi = tile ? start_pos + last_col / H : -1;
+  const int key_hi = tile ? start_pos + (min(ncols, c0 + 16) - 1) / H : -1;
   const int key_lo = (tile && window > 0) ? max(0, start_pos + c0 / H - window + 1) : 0;
   const int c = c0 + col16;
   const int cc = min(c, ncols - 1);
@@ -320,152 +328,80 @@ latent_attention_mfma_shared_kernel(const bf16* __restrict__ q, size_t q_tok, si
 #pragma unroll
   for (int t = 0; t < CT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 
-  constexpr int KSEG = (C + R) / 8;     // pieces of 16 bytes in a key's row
-  constexpr int THREADS = LM_WAVES * MS_WAVE;
-  constexpr int KPT = (32 * KSEG + THREADS - 1) / THREADS, VPT = C * 4 / THREADS;   // pieces a thread carries
-  // A key block is asked for one block ahead, into registers, and its page ids one block before that: while a block is
-  // multiplied the next one is on its way, and no load waits for a look-up.
-  bf16x8 kreg[KPT], vreg[VPT];
-  int pages[2];
+  typedef __attribute__((address_space(3))) void lds_void;
+  typedef const __attribute__((address_space(1))) void global_void;
+  int page0 = 0, page1 = 0;        // the pages of the two 16-key halves of the block to be asked for next
   auto lookup = [&](int base) __attribute__((always_inline)) {
-#pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int kb = base + u * 16;
-      pages[u] = kb <= blk_hi ? __builtin_amdgcn_readfirstlane(table[kb / page_size]) : 0;
-    }
+    page0 = base <= blk_hi ? __builtin_amdgcn_readfirstlane(table[base / page_size]) : 0;
+    page1 = base + 16 <= blk_hi ? __builtin_amdgcn_readfirstlane(table[(base + 16) / page_size]) : 0;
   };
-  auto issue = [&](int base) __attribute__((always_inline)) {
-    size_t row0[2];
+  // Keys past the block's last one come from the null page or from what the page's last user left: their scores are
+  // masked, and their latents zeroed in LDS before use.
+  auto issue = [&](int base, bf16* buf) __attribute__((always_inline)) {
+    const int off0 = base % page_size, off1 = base + 16 <= blk_hi ? (base + 16) % page_size : 0;
+    const size_t row0 = (size_t)page0 * page_size + off0, row1 = (size_t)page1 * page_size + off1;
+    const bf16* vt0 = ct_pages + (size_t)page0 * page_size * C + off0;
+    const bf16* vt1 = ct_pages + (size_t)page1 * page_size * C + off1;
+    int lane_now = lane;       // each load's place is worked out when it is asked for: kept across the loop the places of all
+    asm volatile("" : "+v"(lane_now));     // loads would take the registers that the accumulators need
 #pragma unroll
-    for (int u = 0; u < 2; ++u) row0[u] = (size_t)pages[u] * page_size + (base + u * 16 <= blk_hi ? (base + u * 16) % page_size : 0);
-#pragma unroll
-    for (int j = 0; j < KPT; ++j) {
-      const int seg = threadIdx.x + j * THREADS;
-      if (seg < 32 * KSEG) {
-        const int key = seg / KSEG, piece = seg - key * KSEG;
-        const size_t row = row0[key >> 4] + (key & 15);
-        const bf16* src = piece < C / 8 ? c_pages + row * C + piece * 8 : r_pages + row * R + (piece - C / 8) * 8;
-        kreg[j] = *reinterpret_cast<const bf16x8*>(src);
+    for (int p = 0; p < LOADS; ++p) {
+      const int load = wave + p * WAVES;
+      if ((p + 1) * WAVES <= L::K_LOADS || (p * WAVES < L::K_LOADS && load < L::K_LOADS)) {
+        const int at = load * MS_WAVE + lane_now, key = at / L::KP, place = at - key * L::KP;
+        const int piece = place ^ ((key >> L::SHIFT) & L::MASK);   // (within its group: the latent's pieces stay the latent's)
+        const size_t row = (key < 16 ? row0 : row1) + (key & 15);
+        const bool latent = piece < C / 8;
+        const bf16* from = latent ? c_pages : r_pages;
+        const size_t off = row * (latent ? C : R) + (piece - (latent ? 0 : C / 8)) * 8;
+        __builtin_amdgcn_global_load_lds((global_void*)(from + off), (lds_void*)(buf + (size_t)load * MS_WAVE * 8), 16, 0, 0);
+      } else if ((p + 1) * WAVES <= L::K_LOADS + L::V_LOADS || load < L::K_LOADS + L::V_LOADS) {
+        const int at = (load - L::K_LOADS) * MS_WAVE + lane_now, dim = at >> 2, piece = (at & 3) ^ ((dim >> 2) & 3);
+        const bf16* from = piece < 2 ? vt0 : vt1;
+        const size_t off = (size_t)dim * page_size + (piece & 1) * 8;
+        __builtin_amdgcn_global_load_lds((global_void*)(from + off), (lds_void*)(buf + (size_t)load * MS_WAVE * 8), 16, 0, 0);
       }
     }
-#pragma unroll
-    for (int j = 0; j < VPT; ++j) {
-      const int seg = threadIdx.x + j * THREADS;
-      const int u = seg / (C * 2), rem = seg - u * (C * 2), dim = rem >> 1, piece = rem & 1;
-      const bf16* src = ct_pages + (row0[u] / page_size) * (size_t)page_size * C + (size_t)dim * page_size +
-                        row0[u] % page_size + piece * 8;
-      vreg[j] = *reinterpret_cast<const bf16x8*>(src);
-    }
   };
-  auto commit = [&](int base) __attribute__((always_inline)) {
-#pragma unroll
-    for (int j = 0; j < KPT; ++j) {
-      const int seg = threadIdx.x + j * THREADS;
-      if (seg < 32 * KSEG) {
-        const int key = seg / KSEG, piece = seg - key * KSEG;
-        *reinterpret_cast<bf16x8*>(Ks + key * KROW + piece * 8) = kreg[j];
-      }
-    }
-#pragma unroll
-    for (int j = 0; j < VPT; ++j) {
-      const int seg = threadIdx.x + j * THREADS;
-      const int u = seg / (C * 2), rem = seg - u * (C * 2), dim = rem >> 1, piece = rem & 1;
-      bf16x8 v = vreg[j];
-      // what a reused page still holds past the block's last key must not meet the zero weights
-      const int k0 = base + u * 16 + piece * 8;
-      if (k0 + 7 > blk_hi) {
-#pragma unroll
-        for (int i = 0; i < 8; ++i)
-          if (k0 + i > blk_hi) v[i] = (__bf16)0.0f;
-      }
-      *reinterpret_cast<bf16x8*>(Vs + dim * LS_VROW + u * 16 + piece * 8) = v;
-    }
-  };
-  constexpr bool AHEAD = C <= 256;      // at 512 the accumulators and the query leave no registers to carry a block
+  // this lane's fragment places: key rows of col16 (+ 16), latent rows of col16 (+ 16 t)
+  const int swap = (col16 >> L::SHIFT) & L::MASK;
+  const int k_even = (col16 * L::KP + (kq ^ swap)) * 8, k_odd = (col16 * L::KP + ((kq + 4) ^ swap)) * 8;
+  const int v_swap = (col16 >> 2) & 3;
+  const int v_at0 = 32 * L::KP * 8 + col16 * 32 + (((kq >> 1) ^ v_swap) * 8) + (kq & 1) * 4;
+  const int v_at1 = 32 * L::KP * 8 + col16 * 32 + (((2 + (kq >> 1)) ^ v_swap) * 8) + (kq & 1) * 4;
+
   const int first = (blk_lo / 32) * 32;
   lookup(first);
-  if (AHEAD) {
-    issue(first);
-    if (first + 32 <= blk_hi) lookup(first + 32);
-  }
-  for (int base = first; base <= blk_hi; base += 32) {
-    __syncthreads();     // everyone is done with the block before
-    if (AHEAD) {
-      commit(base);
-    } else {
-      // four pieces in flight at a time, straight into LDS
-      size_t row0[2];
-#pragma unroll
-      for (int u = 0; u < 2; ++u) row0[u] = (size_t)pages[u] * page_size + (base + u * 16 <= blk_hi ? (base + u * 16) % page_size : 0);
-      if (base + 32 <= blk_hi) lookup(base + 32);     // the next block's page ids travel with this block's keys
-      constexpr int G = 4;
-#pragma unroll
-      for (int j0 = 0; j0 < KPT; j0 += G) {
-        bf16x8 t[G];
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-          const int seg = threadIdx.x + (j0 + g) * THREADS;
-          if (j0 + g < KPT && seg < 32 * KSEG) {
-            const int key = seg / KSEG, piece = seg - key * KSEG;
-            const size_t row = row0[key >> 4] + (key & 15);
-            t[g] = *reinterpret_cast<const bf16x8*>(piece < C / 8 ? c_pages + row * C + piece * 8
-                                                                  : r_pages + row * R + (piece - C / 8) * 8);
-          }
-        }
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-          const int seg = threadIdx.x + (j0 + g) * THREADS;
-          if (j0 + g < KPT && seg < 32 * KSEG) {
-            const int key = seg / KSEG, piece = seg - key * KSEG;
-            *reinterpret_cast<bf16x8*>(Ks + key * KROW + piece * 8) = t[g];
-          }
-        }
+  issue(first, ls);
+  lookup(first + 32);
+  int turn = 0;
+  for (int base = first; base <= blk_hi; base += 32, turn ^= 1) {
+    __builtin_amdgcn_s_waitcnt(0x0F70);   // vmcnt(0): this wave's share of the block has landed in LDS
+    __syncthreads();                      // everybody's has, and nobody reads the other buffer any more
+    bf16* buf = ls + (turn ? L::BUFFER : 0);
+    if (base + 31 > blk_hi) {             // what a reused page still holds past the last key must not meet the zero weights
+#pragma unroll 1
+      for (int e = threadIdx.x; e < C * 32; e += WAVES * MS_WAVE) {
+        const int dim = e >> 5, place = e & 31, key = (((place >> 3) ^ ((dim >> 2) & 3)) << 3) + (place & 7);
+        if (base + key > blk_hi) buf[32 * L::KP * 8 + e] = from_float<bf16>(0.f);
       }
-#pragma unroll
-      for (int j0 = 0; j0 < VPT; j0 += G) {
-        bf16x8 t[G];
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-          if (j0 + g < VPT) {
-            const int seg = threadIdx.x + (j0 + g) * THREADS;
-            const int u = seg / (C * 2), rem = seg - u * (C * 2), dim = rem >> 1, piece = rem & 1;
-            t[g] = *reinterpret_cast<const bf16x8*>(ct_pages + (row0[u] / page_size) * (size_t)page_size * C +
-                                                    (size_t)dim * page_size + row0[u] % page_size + piece * 8);
-          }
-        }
-#pragma unroll
-        for (int g = 0; g < G; ++g) {
-          if (j0 + g < VPT) {
-            const int seg = threadIdx.x + (j0 + g) * THREADS;
-            const int u = seg / (C * 2), rem = seg - u * (C * 2), dim = rem >> 1, piece = rem & 1;
-            bf16x8 v = t[g];
-            const int k0 = base + u * 16 + piece * 8;
-            if (k0 + 7 > blk_hi) {
-#pragma unroll
-              for (int i = 0; i < 8; ++i)
-                if (k0 + i > blk_hi) v[i] = (__bf16)0.0f;
-            }
-            *reinterpret_cast<bf16x8*>(Vs + dim * LS_VROW + u * 16 + piece * 8) = v;
-          }
-        }
-      }
+      __syncthreads();
     }
-    __syncthreads();
-    if (AHEAD && base + 32 <= blk_hi) {
-      issue(base + 32);
-      if (base + 64 <= blk_hi) lookup(base + 64);
+    if (base + 32 <= blk_hi) {
+      issue(base + 32, ls + (turn ? 0 : L::BUFFER));
+      lookup(base + 64);
     }
     if (!tile || base > key_hi || base + 31 < key_lo) continue;     // none of this block's keys is the tile's
     f32x4 s[2];
 #pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const bf16* kp = Ks + (u * 16 + col16) * KROW + kq * 8;
-      f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int u = 0; u < 2; ++u) s[u] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int ks = 0; ks < KS_C + KS_R; ++ks)
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kp + ks * 32), qv[ks], acc, 0, 0, 0);
-      s[u] = acc;
-    }
+    for (int ks = 0; ks < KS_C + KS_R; ++ks)
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const bf16* kp = buf + u * 16 * L::KP * 8 + (ks & 1 ? k_odd : k_even) + (ks >> 1) * 64;
+        s[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const bf16x8*>(kp), qv[ks], s[u], 0, 0, 0);
+      }
     float bm = -INFINITY;
 #pragma unroll
     for (int u = 0; u < 2; ++u)
@@ -494,16 +430,16 @@ latent_attention_mfma_shared_kernel(const bf16* __restrict__ q, size_t q_tok, si
       for (int t = 0; t < CT; ++t) o[t] *= corr;
     }
     lsum = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, p, lsum, 0, 0, 0);
-#pragma unroll
-    for (int t = 0; t < CT; ++t) {
-      const bf16* vp = Vs + (t * 16 + col16) * LS_VROW + kq * 4;
-      const bf16x4 a = *reinterpret_cast<const bf16x4*>(vp);
-      const bf16x4 b = *reinterpret_cast<const bf16x4*>(vp + 16);
+    auto value = [&](int t) __attribute__((always_inline)) {
+      const bf16x4 a = *reinterpret_cast<const bf16x4*>(buf + v_at0 + t * 16 * 32);
+      const bf16x4 b = *reinterpret_cast<const bf16x4*>(buf + v_at1 + t * 16 * 32);
       bf16x8 vv;
 #pragma unroll
       for (int i = 0; i < 4; ++i) { vv[i] = a[i]; vv[4 + i] = b[i]; }
-      o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, p, o[t], 0, 0, 0);
-    }
+      return vv;
+    };
+#pragma unroll
+    for (int t = 0; t < CT; ++t) o[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(value(t), p, o[t], 0, 0, 0);
   }
   if (pos < 0) return;
   float l = lsum[0];
@@ -552,26 +488,32 @@ extern "C" int ms_latent_attention_mfma(const void* q, long long q_tok, long lon
   if (num_pages * page_size >= (1ll << 31) || n_requests > 65535) return MS_UNSUPPORTED;
   const long long tiles = ((long long)max_q_len * heads + 15) / 16;
   const float sl = scale * 1.4426950408889634f;
-  // long portions: four neighbouring tiles a block over key blocks staged in LDS (more than the 64 KB a launch may
-  // ask for without more ado, so the kernel's limit is raised once); else a tile's keys over the four waves
-  const size_t shared_lds = ((size_t)32 * (C + R + LS_KPAD) + (size_t)C * LS_VROW) * sizeof(bf16);
-  const bool shared = tiles >= 8 && splits == 1;
-  dim3 grid((unsigned)(shared ? (tiles + LM_WAVES - 1) / LM_WAVES : tiles), n_requests, splits), block(LM_WAVES * MS_WAVE);
+  // long portions: neighbouring tiles over key blocks staged in LDS (more than the 64 KB a launch may ask for without more
+  // ado, so the kernel's limit is raised once), eight tiles a block where that still fills the chip; else a tile's keys over
+  // the four waves of a block
+  const bool staged = tiles >= 8 && splits == 1;
+  const bool wide = staged && (tiles + 7) / 8 * n_requests >= ms_compute_units();
+  const int per = wide ? 8 : (staged ? LM_WAVES : 1);
+  dim3 grid((unsigned)((tiles + per - 1) / per), n_requests, splits), block((wide ? 8 : LM_WAVES) * MS_WAVE);
 #define ARGS                                                                                                            \
       (const bf16*)q, (size_t)q_tok, (size_t)q_head, (const bf16*)c_pages, (const bf16*)r_pages, (const bf16*)ct_pages, \
       block_table, table_stride, table_rows, q_start, context_lens, sink, (bf16*)out, (size_t)out_tok,                  \
       (size_t)out_head, heads, page_size, sl, window
 #define LAUNCH(CC, RR)                                                                                                  \
   do {                                                                                                                  \
-    if (shared) {                                                                                                       \
+    constexpr size_t lds = 2 * Staged<CC, RR>::BUFFER * sizeof(bf16);                                                   \
+    if (staged) {                                                                                                       \
       static bool raised = false;                                                                                       \
       if (!raised) {                                                                                                    \
-        if (hipFuncSetAttribute((const void*)latent_attention_mfma_shared_kernel<CC, RR>,                               \
-                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)shared_lds) != hipSuccess)             \
+        if (hipFuncSetAttribute((const void*)latent_attention_mfma_staged_kernel<CC, RR, LM_WAVES>,                     \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess ||                  \
+            hipFuncSetAttribute((const void*)latent_attention_mfma_staged_kernel<CC, RR, 8>,                            \
+                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)                    \
           return MS_LAUNCH_FAILED;                                                                                      \
         raised = true;                                                                                                  \
       }                                                                                                                 \
-      latent_attention_mfma_shared_kernel<CC, RR><<<grid, block, shared_lds, stream>>>(ARGS);                           \
+      if (wide) latent_attention_mfma_staged_kernel<CC, RR, 8><<<grid, block, lds, stream>>>(ARGS);                     \
+      else latent_attention_mfma_staged_kernel<CC, RR, LM_WAVES><<<grid, block, lds, stream>>>(ARGS);                   \
     } else if (splits > 1) {                                                                                            \
       latent_attention_mfma_kernel<CC, RR, true><<<grid, block, 0, stream>>>(ARGS, part_o, part_ml);                    \
     } else {                                                                                                            \
