@@ -77,7 +77,7 @@ int ms_gemm_panel_splitk(const void* A, long long lda, const void* W, long long 
 // as epilogue 1; K a multiple of 64 (ms_gemm_tiled_force: measurements, 0 leaves the choice of tile, 1 to 5 force one;
 // ms_gemm_tiled_pays: whether the gated product is faster here than as library product and activation kernel).
 int ms_gemm_tiled(const void* A, long long lda, const void* W, long long ldw, void* out, long long ldo, int M, int N,
-                  int K, int epilogue, hipStream_t stream);
+                  int K, int epilogue, float limit, float alpha, hipStream_t stream);
 void ms_gemm_tiled_force(int tile);
 void ms_gemm_tiled_force_xcd_split(int xm);   // measurements: rows of XCDs over the tiles (1, 2, 4, 8); 0 leaves the choice
 int ms_gemm_tiled_pays(int M, int N, int K);
@@ -258,14 +258,16 @@ int ms_moe_align(const int* ids, int n_items, int n_experts, int tile, int tiles
 int ms_gemm_tiled_grouped_rows();
 int ms_gemm_tiled_grouped(const void* A, long long lda, const void* W, const int* rows, const int* tile_expert, void* out,
                           long long ldo, int tiles, int tile_rows, int N, int K, int in_div, int out_scatter, int act,
-                          int out_dtype, hipStream_t stream);
+                          float limit, float alpha, int out_dtype, hipStream_t stream);
 
 int ms_grouped_gemm_mfma_ok(int K, long long in_stride, long long out_stride, int tile, int dtype, int out_dtype);
 // for every tile t with an expert e and each of its rows i (flat position p = t * tile + i, item = rows[p] >= 0):
-// out[out_scatter ? item : p] = act(w[e] . in[in_div ? item / in_div : p]); w [experts, n_out, K]
+// out[out_scatter ? item : p] = act(w[e] . in[in_div ? item / in_div : p]); w [experts, n_out, K]; act 0: none, 1: the exact
+// gelu, 2: the clamped gate (limit, alpha) over interleaved gate and up rows of w, out [., n_out / 2] bfloat16 (the matrix
+// cores' tiles alone: MS_UNSUPPORTED elsewhere)
 int ms_grouped_gemm(const void* in, long long in_stride, const void* w, const int* rows, const int* tile_expert, void* out,
                     long long out_stride, int tiles, int tile, int n_out, int K, int in_div, int out_scatter, int act,
-                    int dtype, int out_dtype, hipStream_t stream);
+                    float limit, float alpha, int dtype, int out_dtype, hipStream_t stream);
 int ms_moe_combine(const float* part, const int* ids, const float* weights, const void* h, long long h_stride,
                    const void* shared, int shared_dtype, const float* gate, long long gate_stride, float* out,
                    int n_tokens, int top, int n_experts, int hidden, int dtype, hipStream_t stream);   // weights null: all 1; gate null: shared added as it is

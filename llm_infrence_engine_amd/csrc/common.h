@@ -52,6 +52,29 @@ __device__ __forceinline__ float fast_silu(float g) {
   return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * g));
 }
 
+// The clamped gate: g = min(g, limit), u = clamp(u, -limit, limit), g * sigmoid(alpha g) * (u + 1), for results that are
+// rounded to bfloat16.
+__device__ __forceinline__ float fast_clamped_glu(float g, float u, float limit, float alpha) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * alpha * g)) * (u + 1.0f);
+}
+
+__device__ __forceinline__ float relu_squared(float z) { const float r = fmaxf(z, 0.f); return r * r; }
+
+// Epilogues of the few-rows products (csrc/gemm_skinny.hip, gemm_stream.hip, gemm_panel.hip):
+//   EPI_STORE     out[M, N] = product (+ bias)
+//   EPI_SWIGLU    out[M, N / 2] = silu(gate) * up over interleaved rows of W (no bias)
+//   EPI_RESIDUAL  out[M, N] += product (+ bias), float
+//   EPI_RELU2     out[M, N] = max(product (+ bias), 0)^2
+//   EPI_CLAMPED   as EPI_SWIGLU with the clamped gate; `bias` points at its two numbers, limit and alpha
+enum { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 3, EPI_RELU2 = 5, EPI_CLAMPED = 6 };
+constexpr bool ms_gated(int epi) { return epi == EPI_SWIGLU || epi == EPI_CLAMPED; }
+template <int EPI> __device__ __forceinline__ float ms_gate_value(float g, float u, const float* __restrict__ numbers) {
+  return EPI == EPI_CLAMPED ? fast_clamped_glu(g, u, numbers[0], numbers[1]) : fast_silu(g) * u;
+}
+template <int EPI> __device__ __forceinline__ float ms_store_value(float v) { return EPI == EPI_RELU2 ? relu_squared(v) : v; }
+
 // sin and cos of a rotation angle for bfloat16 results: three-part Cody-Waite reduction by pi/2 (the first
 // two parts have 11 bits, so n * part is exact for |x| < 2^13 * pi/2) and short polynomials on [-pi/4, pi/4];
 // absolute error ~2e-7.  Larger angles take the library routine.

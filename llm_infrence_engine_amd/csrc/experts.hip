@@ -2,7 +2,8 @@
 //   route    per token: softmax over the router's outputs, the `top` largest of (score + correction), their scores;
 //            optionally inside the best groups of neighbouring outputs only, and with the scores divided by their sum
 //   align    rows (token, choice) grouped by expert into tiles of TILE rows, each tile of one expert
-//   grouped  out[row] = act(W[expert of the row's tile] . in[row]) for every tile, gathered / scattered by the rows' list
+//   grouped  out[row] = act(W[expert of the row's tile] . in[row]) for every tile, gathered / scattered by the rows' list;
+//            act: none, the exact gelu, or (matrix cores) the clamped gate over interleaved gate and up features
 //   combine  out[n] = sum_j weight[n, j] * (expert j's row, or the token's input for an identity expert)
 //                     (+ sigmoid(gate[n]) * shared[n], or + shared[n])
 // and two activations: the exact gelu, z/2 (1 + erf(z / sqrt 2)), and the square of relu.  Router scores, weights and all sums are float.
@@ -55,6 +56,8 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
 #pragma unroll
   for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
     const int e = lane + i * MS_WAVE;
+    s[i] = c[i] = -INFINITY;
+    if (i * MS_WAVE >= n_out) continue;        // (here and below: pieces past the outputs cost nothing)
     s[i] = e < n_out ? z[e] : -INFINITY;
     big = fmaxf(big, s[i]);
   }
@@ -63,6 +66,7 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
 #pragma unroll
   for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
     const int e = lane + i * MS_WAVE;
+    if (i * MS_WAVE >= n_out) continue;
     s[i] = e < n_out ? (sigmoid_scores ? 1.0f / (1.0f + expf(-s[i])) : expf(s[i] - big)) : 0.f;
     sum += s[i];
   }
@@ -71,6 +75,7 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
 #pragma unroll
   for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
     const int e = lane + i * MS_WAVE;
+    if (i * MS_WAVE >= n_out) continue;
     s[i] *= inv;
     c[i] = e < n_out ? s[i] + (correction ? correction[e] : 0.f) : -INFINITY;
   }
@@ -113,6 +118,7 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
 #pragma unroll
     for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i) {
       const int e = lane + i * MS_WAVE;
+      if (i * MS_WAVE >= n_out) continue;
       if (c[i] > bv) { bv = c[i]; be = e; bs = s[i]; }   // a lane's indices rise with i: the first maximum stays
     }
 #pragma unroll
@@ -126,7 +132,7 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
     total += bs;
 #pragma unroll
     for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
-      if (lane + i * MS_WAVE == be) c[i] = -INFINITY;
+      if (i * MS_WAVE < n_out && lane + i * MS_WAVE == be) c[i] = -INFINITY;
   }
   if (lane < top) weights[(size_t)n * top + lane] = normalise ? my_weight / (total + 1e-20f) : my_weight;
 }
@@ -238,7 +244,7 @@ template <int NT, typename TO>
 __global__ void __launch_bounds__(256)
 grouped_gemm_mfma_kernel(const bf16* __restrict__ in, size_t in_stride, const bf16* __restrict__ w,
                          const int* __restrict__ rows, const int* __restrict__ tile_expert, TO* __restrict__ out,
-                         size_t out_stride, int n_out, int K, int in_div, int out_scatter, int act) {
+                         size_t out_stride, int n_out, int K, int in_div, int out_scatter, int act, float limit, float alpha) {
   constexpr int TM = 16 * NT;
   const int tile = blockIdx.y;
   const int e = tile_expert[tile];
@@ -292,6 +298,13 @@ grouped_gemm_mfma_kernel(const bf16* __restrict__ in, size_t in_stride, const bf
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       const int f = f0 + u * 16 + kq * 4;
+      if (act == 2) {      // two pairs of gate and up
+#pragma unroll
+        for (int p = 0; p < 2; ++p)
+          if (f + 2 * p + 1 < n_out)
+            out[dst * out_stride + f / 2 + p] = from_float<TO>(fast_clamped_glu(acc[u][t][2 * p], acc[u][t][2 * p + 1], limit, alpha));
+        continue;
+      }
       TO* op = out + dst * out_stride + f;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -314,7 +327,8 @@ template <typename TO>
 __global__ void __launch_bounds__(256, 2)
 grouped_gemm_mfma_wide_kernel(const bf16* __restrict__ in, size_t in_stride, const bf16* __restrict__ w,
                               const int* __restrict__ rows, const int* __restrict__ tile_expert, TO* __restrict__ out,
-                              size_t out_stride, int n_out, int K, int in_div, int out_scatter, int act) {
+                              size_t out_stride, int n_out, int K, int in_div, int out_scatter, int act, float limit,
+                              float alpha) {
   __shared__ __align__(16) bf16 Bs[2][GW_TM][GW_KS + GW_PAD];
   __shared__ int s_item[GW_TM];
   const int tile = blockIdx.y;
@@ -403,6 +417,13 @@ grouped_gemm_mfma_wide_kernel(const bf16* __restrict__ in, size_t in_stride, con
 #pragma unroll
     for (int u = 0; u < GW_FT; ++u) {
       const int f = f0 + u * 16 + kq * 4;
+      if (act == 2) {      // two pairs of gate and up
+#pragma unroll
+        for (int p = 0; p < 2; ++p)
+          if (f + 2 * p + 1 < n_out)
+            out[dst * out_stride + f / 2 + p] = from_float<TO>(fast_clamped_glu(acc[u][t][2 * p], acc[u][t][2 * p + 1], limit, alpha));
+        continue;
+      }
       TO* op = out + dst * out_stride + f;
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -498,13 +519,15 @@ extern "C" int ms_grouped_gemm_mfma_ok(int K, long long in_stride, long long out
 
 extern "C" int ms_grouped_gemm(const void* in, long long in_stride, const void* w, const int* rows, const int* tile_expert,
                                void* out, long long out_stride, int tiles, int tile, int n_out, int K, int in_div,
-                               int out_scatter, int act, int dtype, int out_dtype, hipStream_t stream) {
+                               int out_scatter, int act, float limit, float alpha, int dtype, int out_dtype,
+                               hipStream_t stream) {
   if (tiles <= 0) return MS_OK;
-  if (n_out <= 0 || K <= 0 || in_div < 0) return MS_BAD_ARG;
+  if (n_out <= 0 || K <= 0 || in_div < 0 || (act == 2 && n_out % 2)) return MS_BAD_ARG;
   if (tile == ms_gemm_tiled_grouped_rows() || (tile * 2 == ms_gemm_tiled_grouped_rows() && K % 64 == 0 && dtype == MS_BF16)) {
     // wide tiles with K a multiple of 64: the tiled kernel, operands from memory straight to LDS
     const int rc = dtype == MS_BF16 ? ms_gemm_tiled_grouped(in, in_stride, w, rows, tile_expert, out, out_stride, tiles,
-                                                            tile, n_out, K, in_div, out_scatter, act, out_dtype, stream)
+                                                            tile, n_out, K, in_div, out_scatter, act, limit, alpha,
+                                                            out_dtype, stream)
                                     : MS_UNSUPPORTED;
     if (rc != MS_UNSUPPORTED || tile == ms_gemm_tiled_grouped_rows()) return rc;
   }
@@ -517,11 +540,11 @@ extern "C" int ms_grouped_gemm(const void* in, long long in_stride, const void* 
 #define LAUNCH_W(TO)                                                                                                  \
   grouped_gemm_mfma_wide_kernel<TO><<<grid, block, 0, stream>>>((const bf16*)in, (size_t)in_stride, (const bf16*)w, rows, \
                                                                 tile_expert, (TO*)out, (size_t)out_stride, n_out, K,  \
-                                                                in_div, out_scatter, act)
+                                                                in_div, out_scatter, act, limit, alpha)
 #define LAUNCH_M(NT, TO)                                                                                              \
   grouped_gemm_mfma_kernel<NT, TO><<<grid, block, 0, stream>>>((const bf16*)in, (size_t)in_stride, (const bf16*)w, rows, \
                                                                tile_expert, (TO*)out, (size_t)out_stride, n_out, K,   \
-                                                               in_div, out_scatter, act)
+                                                               in_div, out_scatter, act, limit, alpha)
     if (tile == GM && out_dtype == MS_F32) LAUNCH_M(1, float);
     else if (tile == GM) LAUNCH_M(1, bf16);
     else if (out_dtype == MS_F32) LAUNCH_W(float);
@@ -530,7 +553,7 @@ extern "C" int ms_grouped_gemm(const void* in, long long in_stride, const void* 
 #undef LAUNCH_W
     return ms_launch_status();
   }
-  if (tile != GM) return MS_UNSUPPORTED;
+  if (tile != GM || act == 2) return MS_UNSUPPORTED;
   const int cb = (n_out + GN - 1) / GN;
   if (cb > 65535) return MS_UNSUPPORTED;
   dim3 grid(tiles, cb), block(256);

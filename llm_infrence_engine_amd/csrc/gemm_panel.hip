@@ -29,7 +29,6 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 typedef __attribute__((ext_vector_type(4))) unsigned u32x4;   // a 16-byte piece: 8 bfloat16
 
-enum { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 3 };
 
 constexpr int WAVES = 16;       // waves of a block
 constexpr int BATCH = 4;        // panel loads a wave has in flight
@@ -129,7 +128,7 @@ __device__ __forceinline__ void finish_tile(const f32x4* sum, int n0, int M, int
                                             TO* __restrict__ out, size_t ldo, const float* inv_rms, int col, int kq) {
   const int nb = n0 + kq * 4;
   f32x4 bv = {0.f, 0.f, 0.f, 0.f};
-  if (bias && EPI != EPI_SWIGLU) {
+  if (bias && !ms_gated(EPI)) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) if (nb + r < N) bv[r] = bias[nb + r];
   }
@@ -139,18 +138,18 @@ __device__ __forceinline__ void finish_tile(const f32x4* sum, int n0, int M, int
     if (m >= M) continue;
     f32x4 v = sum[tt];
     if (NORM) v *= inv_rms[m];
-    if (EPI == EPI_SWIGLU) {
+    if (ms_gated(EPI)) {
       // rows nb, nb+1 are (gate, up) of feature nb/2; rows nb+2, nb+3 of feature nb/2 + 1
 #pragma unroll
       for (int p = 0; p < 2; ++p)
-        if (nb + 2 * p + 1 < N) out[(size_t)m * ldo + nb / 2 + p] = from_float<TO>(fast_silu(v[2 * p]) * v[2 * p + 1]);
+        if (nb + 2 * p + 1 < N) out[(size_t)m * ldo + nb / 2 + p] = from_float<TO>(ms_gate_value<EPI>(v[2 * p], v[2 * p + 1], bias));
     } else {
       TO* o = out + (size_t)m * ldo + nb;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         if (nb + r >= N) continue;
         if (EPI == EPI_RESIDUAL) o[r] = from_float<TO>(to_float(o[r]) + v[r] + bv[r]);
-        else o[r] = from_float<TO>(v[r] + bv[r]);
+        else o[r] = from_float<TO>(ms_store_value<EPI>(v[r] + bv[r]));
       }
     }
   }
@@ -566,6 +565,7 @@ int run_splitk(const bf16* A, size_t lda, const bf16* W, size_t ldw, const float
 // epilogue 0: out[M,N] (out_dtype float or bfloat16) = product + bias
 // epilogue 1: out[M,N/2] bfloat16 = silu(gate) * up over interleaved rows of W (no bias)
 // epilogue 3: out[M,N] float += product + bias (not with norm)
+// epilogues 5, 6: bfloat16, not with norm, see common.h
 // MS_UNSUPPORTED for shapes it does not take (the caller then uses ms_gemm_skinny): with any_shape = 0 all but
 // those it is the faster kernel for; with any_shape = 1 (tests, measurements) only those it cannot compute
 // (more than 63 tiles of W to a block, 47 with more than 48 rows, when the rows have to go through LDS in chunks).
@@ -588,6 +588,14 @@ extern "C" int ms_gemm_panel(const void* A, long long lda, const int* rows, cons
   if (epilogue == EPI_SWIGLU) {
     if (N % 2 || ldo < N / 2 || out_dtype != MS_BF16 || bias) return MS_BAD_ARG;
     if (norm) RUN(EPI_SWIGLU, bf16, true); else RUN(EPI_SWIGLU, bf16, false);
+  }
+  if (epilogue == EPI_CLAMPED) {
+    if (N % 2 || ldo < N / 2 || out_dtype != MS_BF16 || norm || !bias) return MS_BAD_ARG;
+    RUN(EPI_CLAMPED, bf16, false);
+  }
+  if (epilogue == EPI_RELU2) {
+    if (ldo < N || out_dtype != MS_BF16 || norm) return MS_BAD_ARG;
+    RUN(EPI_RELU2, bf16, false);
   }
   if (epilogue == EPI_RESIDUAL) {
     if (ldo < N || out_dtype != MS_F32 || norm) return MS_BAD_ARG;

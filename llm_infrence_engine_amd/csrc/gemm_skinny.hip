@@ -25,7 +25,6 @@ namespace {
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 
-enum { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 3 };
 
 constexpr int UNIT = 2;   // rows of W are dealt out in units of two (a gate/up pair)
 
@@ -82,7 +81,7 @@ gemm_skinny_kernel(const void* __restrict__ Av, size_t lda, const bf16* __restri
   for (int u = 0; u < NTILE; ++u) {
     const int nb = n0 + u * 16 + kq * 4;
     bv[u] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (bias && EPI != EPI_SWIGLU) {
+    if (bias && !ms_gated(EPI)) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) if (nb + r < n1) bv[u][r] = bias[nb + r];
     }
@@ -175,13 +174,13 @@ gemm_skinny_kernel(const void* __restrict__ Av, size_t lda, const bf16* __restri
       const int m = m0 + t * 16 + col;
       const int nb = n0 + u * 16 + kq * 4;
       if (m >= M) continue;
-      if (EPI == EPI_SWIGLU) {
+      if (ms_gated(EPI)) {
         // rows nb, nb+1 are (gate, up) of feature nb/2; rows nb+2, nb+3 of feature nb/2 + 1
 #pragma unroll
         for (int p = 0; p < 2; ++p) {
           if (nb + 2 * p + 1 < n1) {
             const float g = sum[2 * p], up = sum[2 * p + 1];
-            out[(size_t)m * ldo + nb / 2 + p] = from_float<TO>(fast_silu(g) * up);
+            out[(size_t)m * ldo + nb / 2 + p] = from_float<TO>(ms_gate_value<EPI>(g, up, bias));
           }
         }
       } else {
@@ -190,7 +189,7 @@ gemm_skinny_kernel(const void* __restrict__ Av, size_t lda, const bf16* __restri
         // against 64 us)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-          if (nb + r < n1) o[r] = from_float<TO>(sum[r] + bv[u][r] + pre[u][t][r]);
+          if (nb + r < n1) o[r] = from_float<TO>(ms_store_value<EPI>(sum[r] + bv[u][r] + pre[u][t][r]));
         }
       }
     }
@@ -264,6 +263,7 @@ extern "C" void ms_gemm_skinny_force(int ntile, int waves, int token_groups) {
 // epilogue 0: out[M,N] (out_dtype float or bfloat16) = product + bias
 // epilogue 1: out[M,N/2] bfloat16 = silu(gate) * up over interleaved rows of W (no bias)
 // epilogue 3: out[M,N] float += product + bias
+// epilogues 5, 6: bfloat16, see common.h
 extern "C" int ms_gemm_skinny(const void* A, long long lda, const void* W, long long ldw, const float* bias, void* out,
                               long long ldo, int M, int N, int K, int epilogue, int out_dtype, hipStream_t stream) {
   if (M <= 0 || N <= 0) return MS_OK;
@@ -288,6 +288,14 @@ extern "C" int ms_gemm_skinny(const void* A, long long lda, const void* W, long 
   if (epilogue == EPI_SWIGLU) {
     if (N % 2 || ldo < N / 2 || out_dtype != MS_BF16 || bias) return MS_BAD_ARG;
     return launch_mt<EPI_SWIGLU, bf16, false>(A, lda, w, ldw, nullptr, (bf16*)out, ldo, M, N, K, stream);
+  }
+  if (epilogue == EPI_CLAMPED) {
+    if (N % 2 || ldo < N / 2 || out_dtype != MS_BF16 || !bias) return MS_BAD_ARG;
+    return launch_mt<EPI_CLAMPED, bf16, false>(A, lda, w, ldw, bias, (bf16*)out, ldo, M, N, K, stream);
+  }
+  if (epilogue == EPI_RELU2) {
+    if (ldo < N || out_dtype != MS_BF16) return MS_BAD_ARG;
+    return launch_mt<EPI_RELU2, bf16, false>(A, lda, w, ldw, bias, (bf16*)out, ldo, M, N, K, stream);
   }
   if (epilogue == EPI_RESIDUAL) {
     if (ldo < N || out_dtype != MS_F32) return MS_BAD_ARG;

@@ -29,7 +29,6 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 typedef __attribute__((ext_vector_type(4))) unsigned u32x4;   // a 16-byte piece: 8 bfloat16
 
-enum { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_RESIDUAL = 3 };
 
 // id / parts for the small numbers that occur here (id < 4096, parts <= 16) by a multiplication: dividing by a
 // run-time value costs some twenty instructions even when both are the same for the whole wave, and the item
@@ -78,7 +77,7 @@ gemm_stream_kernel(const void* __restrict__ Av, size_t lda, const bf16* __restri
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         if (nb + r >= N) continue;
-        if (bias && EPI != EPI_SWIGLU) bv[r] = bias[nb + r];
+        if (bias && !ms_gated(EPI)) bv[r] = bias[nb + r];
         if (EPI == EPI_RESIDUAL) pre[r] = reinterpret_cast<const float*>(out)[(size_t)col * ldo + nb + r];
       }
     }
@@ -234,20 +233,20 @@ gemm_stream_kernel(const void* __restrict__ Av, size_t lda, const bf16* __restri
     const int f = u * 16 + kq * 4;
     const int nb = r0 + f;
     if (col >= M || f >= R) continue;
-    if (EPI == EPI_SWIGLU) {
+    if (ms_gated(EPI)) {
       // rows nb, nb+1 are (gate, up) of feature nb/2; rows nb+2, nb+3 of feature nb/2 + 1
 #pragma unroll
       for (int p = 0; p < 2; ++p) {
         if (nb + 2 * p + 1 < N) {
           const float g = sum[2 * p], up = sum[2 * p + 1];
-          out[(size_t)col * ldo + nb / 2 + p] = from_float<TO>(fast_silu(g) * up);
+          out[(size_t)col * ldo + nb / 2 + p] = from_float<TO>(ms_gate_value<EPI>(g, up, bias));
         }
       }
     } else {
       TO* o = out + (size_t)col * ldo + nb;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        if (nb + r < N) o[r] = from_float<TO>(sum[r] + bv[r] + pre[r]);
+        if (nb + r < N) o[r] = from_float<TO>(ms_store_value<EPI>(sum[r] + bv[r] + pre[r]));
       }
     }
   }
@@ -316,6 +315,7 @@ int plan(const void* A, size_t lda, const bf16* W, size_t ldw, const float* bias
 // epilogue 0: out[M,N] (out_dtype float or bfloat16) = product + bias
 // epilogue 1: out[M,N/2] bfloat16 = silu(gate) * up over interleaved rows of W (no bias)
 // epilogue 3: out[M,N] float += product + bias (not with norm)
+// epilogues 5, 6: bfloat16, not with norm, see common.h
 // MS_UNSUPPORTED for shapes it does not take (the caller then uses ms_gemm_skinny): with any_shape = 0 all but
 // those it is the faster kernel for; with any_shape = 1 (tests, measurements) only those it cannot compute.
 extern "C" int ms_gemm_stream(const void* A, long long lda, const int* rows, const float* norm_w, float eps,
@@ -337,6 +337,14 @@ extern "C" int ms_gemm_stream(const void* A, long long lda, const int* rows, con
   if (epilogue == EPI_SWIGLU) {
     if (N % 2 || ldo < N / 2 || out_dtype != MS_BF16 || bias) return MS_BAD_ARG;
     if (norm) RUN(EPI_SWIGLU, bf16, true); else RUN(EPI_SWIGLU, bf16, false);
+  }
+  if (epilogue == EPI_CLAMPED) {
+    if (N % 2 || ldo < N / 2 || out_dtype != MS_BF16 || norm || !bias) return MS_BAD_ARG;
+    RUN(EPI_CLAMPED, bf16, false);
+  }
+  if (epilogue == EPI_RELU2) {
+    if (ldo < N || out_dtype != MS_BF16 || norm) return MS_BAD_ARG;
+    RUN(EPI_RELU2, bf16, false);
   }
   if (epilogue == EPI_RESIDUAL) {
     if (ldo < N || out_dtype != MS_F32 || norm) return MS_BAD_ARG;

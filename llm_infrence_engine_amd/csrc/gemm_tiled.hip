@@ -23,7 +23,9 @@ namespace {
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 typedef __attribute__((ext_vector_type(4))) float f32x4;
 
-enum { EPI_STORE = 0, EPI_SWIGLU = 1, EPI_QKV = 2, EPI_GROUPED = 3, EPI_GEGLU = 4 };
+// beside the epilogues of common.h (without EPI_RESIDUAL): the q/k/v product's, the grouped product's, and EPI_SWIGLU with
+// the tanh form of the gelu for the silu
+enum { EPI_QKV = 2, EPI_GROUPED = 7, EPI_GEGLU = 4 };
 
 // the gate's activation of a gated epilogue: g * sigmoid(g), or the tanh form of the gelu with the tanh as
 // 1 - 2 / (2^(2 y log2 e) + 1) through the hardware's exp2 and reciprocal (the result is rounded to bfloat16)
@@ -45,7 +47,8 @@ struct GroupedRows {
   size_t expert_stride;     // elements between two experts' matrices
   int in_div;               // > 0: row p of the product reads A[item / in_div]; 0: A[p]
   int out_scatter;          // the result of row p goes to out[item] (else out[p])
-  int act;                  // 1: the exact gelu of the product
+  int act;                  // 1: the exact gelu of the product; 2: the clamped gate over interleaved features
+  float limit, alpha;       // of the clamped gate (EPI_CLAMPED too)
 };
 
 __device__ __forceinline__ float tiled_gelu_erf(float z) { return 0.5f * z * (1.0f + erff(z * 0.70710678118654752440f)); }
@@ -299,19 +302,32 @@ gemm_tiled_kernel(const bf16* __restrict__ A, size_t lda, const bf16* __restrict
   for (int j = 0; j < TT; ++j) {
     const int m = m0 + wt * TT * 16 + j * 16 + col;
     if (m >= M) continue;
-    if (EPI == EPI_SWIGLU || EPI == EPI_GEGLU) {   // features 2g, 2g + 1 are gate g and up g: 2 FT outputs from o0 on
+    if (ms_gated(EPI) || EPI == EPI_GEGLU) {   // features 2g, 2g + 1 are gate g and up g: 2 FT outputs from o0 on
       const int o0 = f0 / 2, n_out = N / 2;
       float v[2 * FT];
 #pragma unroll
       for (int i = 0; i < FT; ++i) {
-        v[2 * i] = gate_act<EPI>(acc[i][j][0]) * acc[i][j][1];
-        v[2 * i + 1] = gate_act<EPI>(acc[i][j][2]) * acc[i][j][3];
+        if (EPI == EPI_CLAMPED) {
+          v[2 * i] = fast_clamped_glu(acc[i][j][0], acc[i][j][1], grp.limit, grp.alpha);
+          v[2 * i + 1] = fast_clamped_glu(acc[i][j][2], acc[i][j][3], grp.limit, grp.alpha);
+        } else {
+          v[2 * i] = gate_act<EPI>(acc[i][j][0]) * acc[i][j][1];
+          v[2 * i + 1] = gate_act<EPI>(acc[i][j][2]) * acc[i][j][3];
+        }
       }
       store_run<2 * FT>(reinterpret_cast<bf16*>(out) + (size_t)m * ldo + o0, v, n_out - o0);
     } else if (EPI == EPI_GROUPED) {
       const int item = grp.rows[m];
       if (item < 0) continue;
       const size_t row = grp.out_scatter ? (size_t)item : (size_t)m;
+      if (sizeof(TO) == 2 && grp.act == 2) {      // gate and up of feature f0 / 2 + g
+        float v[2 * FT];
+#pragma unroll
+        for (int g = 0; g < 2 * FT; ++g)
+          v[g] = fast_clamped_glu(acc[g >> 1][j][2 * (g & 1)], acc[g >> 1][j][2 * (g & 1) + 1], grp.limit, grp.alpha);
+        store_run<2 * FT>(reinterpret_cast<bf16*>(out) + row * ldo + f0 / 2, v, (N - f0) / 2);
+        continue;
+      }
       float v[4 * FT];
 #pragma unroll
       for (int g = 0; g < 4 * FT; ++g) v[g] = grp.act ? tiled_gelu_erf(acc[g >> 2][j][g & 3]) : acc[g >> 2][j][g & 3];
@@ -320,7 +336,7 @@ gemm_tiled_kernel(const bf16* __restrict__ A, size_t lda, const bf16* __restrict
     } else {
       float v[4 * FT];
 #pragma unroll
-      for (int g = 0; g < 4 * FT; ++g) v[g] = acc[g >> 2][j][g & 3];
+      for (int g = 0; g < 4 * FT; ++g) v[g] = ms_store_value<EPI>(acc[g >> 2][j][g & 3]);
       store_run<4 * FT>(reinterpret_cast<bf16*>(out) + (size_t)m * ldo + f0, v, N - f0);
     }
   }
@@ -339,7 +355,7 @@ int choose_xcd_split(int M) {
 
 template <int WF, int WT, int FT, int TT, int EPI, typename TO>
 int launch(const bf16* A, size_t lda, const bf16* W, size_t ldw, TO* out, size_t ldo, int M, int N, int K,
-           hipStream_t stream, const QkvEpilogue& qkv = QkvEpilogue{}) {
+           hipStream_t stream, const QkvEpilogue& qkv = QkvEpilogue{}, const GroupedRows& grp = GroupedRows{}) {
   constexpr int BN = WF * FT * 16, BM = WT * TT * 16;
   constexpr size_t lds = 2 * (size_t)(BN + BM) * PITCH * sizeof(bf16);
   static bool raised = false;   // once per instantiation: allow more dynamic LDS than the default 64 KB
@@ -354,7 +370,7 @@ int launch(const bf16* A, size_t lda, const bf16* W, size_t ldw, TO* out, size_t
   const long long blocks = 8LL * ((m_tiles + xm - 1) / xm) * ((n_tiles + 8 / xm - 1) / (8 / xm));
   if (blocks > 0x7fffffffLL) return MS_UNSUPPORTED;
   gemm_tiled_kernel<WF, WT, FT, TT, EPI, TO><<<dim3((unsigned)blocks), dim3(WF * WT * MS_WAVE), lds, stream>>>(
-      A, lda, W, ldw, out, ldo, M, N, K, m_tiles, n_tiles, xm, qkv, GroupedRows{});
+      A, lda, W, ldw, out, ldo, M, N, K, m_tiles, n_tiles, xm, qkv, grp);
   return ms_launch_status();
 }
 
@@ -436,14 +452,18 @@ extern "C" int ms_gemm_tiled_pays(int M, int N, int K) {
 
 // A bfloat16 [M, lda], W bfloat16 [N, ldw] (rows of K, K a multiple of 64), out bfloat16.
 // epilogue 0: out[M, N] = product;  epilogue 1: out[M, N / 2] = silu(gate) * up over interleaved rows of W;
-// epilogue 4: the same with the tanh form of the gelu for the silu.
+// epilogue 4: the same with the tanh form of the gelu for the silu; epilogue 5: max(product, 0)^2; epilogue 6: as 1 with the
+// clamped gate (limit, alpha).
 extern "C" int ms_gemm_tiled(const void* A, long long lda, const void* W, long long ldw, void* out, long long ldo, int M,
-                             int N, int K, int epilogue, hipStream_t stream) {
+                             int N, int K, int epilogue, float limit, float alpha, hipStream_t stream) {
   if (M <= 0 || N <= 0) return MS_OK;
   if (K <= 0 || K % BK || lda % 8 || ldw % 8 || lda < K || ldw < K) return MS_UNSUPPORTED;
   if (((uintptr_t)A | (uintptr_t)W) % 16) return MS_UNSUPPORTED;
-  const bool gated = epilogue == EPI_SWIGLU || epilogue == EPI_GEGLU;
-  if (gated ? (N % 2 || ldo < N / 2) : (epilogue != EPI_STORE || ldo < N)) return MS_BAD_ARG;
+  const bool gated = ms_gated(epilogue) || epilogue == EPI_GEGLU;
+  if (gated ? (N % 2 || ldo < N / 2) : ((epilogue != EPI_STORE && epilogue != EPI_RELU2) || ldo < N)) return MS_BAD_ARG;
+  GroupedRows numbers{};
+  numbers.limit = limit;
+  numbers.alpha = alpha;
   const bf16* a = (const bf16*)A;
   const bf16* w = (const bf16*)W;
   bf16* o = (bf16*)out;
@@ -451,6 +471,8 @@ extern "C" int ms_gemm_tiled(const void* A, long long lda, const void* W, long l
   if (tile == 0) tile = choose_tile(M, N, K).tile;
 #define GO(WF, WT, FT, TT) return epilogue == EPI_SWIGLU ? launch<WF, WT, FT, TT, EPI_SWIGLU, bf16>(a, lda, w, ldw, o, ldo, M, N, K, stream) \
                                 : epilogue == EPI_GEGLU ? launch<WF, WT, FT, TT, EPI_GEGLU, bf16>(a, lda, w, ldw, o, ldo, M, N, K, stream)  \
+                                : epilogue == EPI_RELU2 ? launch<WF, WT, FT, TT, EPI_RELU2, bf16>(a, lda, w, ldw, o, ldo, M, N, K, stream)  \
+                                : epilogue == EPI_CLAMPED ? launch<WF, WT, FT, TT, EPI_CLAMPED, bf16>(a, lda, w, ldw, o, ldo, M, N, K, stream, QkvEpilogue{}, numbers)  \
                                                         : launch<WF, WT, FT, TT, EPI_STORE, bf16>(a, lda, w, ldw, o, ldo, M, N, K, stream)
   if (tile == 1) GO(2, 4, 8, 4);   // 256 x 256
   if (tile == 3) GO(1, 4, 4, 1);   // 64 x 64, four waves
@@ -467,14 +489,15 @@ extern "C" int ms_gemm_tiled(const void* A, long long lda, const void* W, long l
 extern "C" int ms_gemm_tiled_grouped_rows() { return 4 * GROUPED_TT * 16; }
 extern "C" int ms_gemm_tiled_grouped(const void* A, long long lda, const void* W, const int* rows, const int* tile_expert,
                                      void* out, long long ldo, int tiles, int tile_rows, int N, int K, int in_div,
-                                     int out_scatter, int act, int out_dtype, hipStream_t stream) {
+                                     int out_scatter, int act, float limit, float alpha, int out_dtype, hipStream_t stream) {
   if (tiles <= 0 || N <= 0) return MS_OK;
-  if (K <= 0 || K % BK || lda % 8 || lda < K || ldo < N || in_div < 0) return MS_UNSUPPORTED;
+  if (act == 2 && (N % 2 || out_dtype != MS_BF16)) return MS_BAD_ARG;
+  if (K <= 0 || K % BK || lda % 8 || lda < K || ldo < (act == 2 ? N / 2 : N) || in_div < 0) return MS_UNSUPPORTED;
   if (((uintptr_t)A | (uintptr_t)W) % 16) return MS_UNSUPPORTED;
   const bool whole = tile_rows == ms_gemm_tiled_grouped_rows();
   if (!whole && tile_rows * 2 != ms_gemm_tiled_grouped_rows()) return MS_UNSUPPORTED;
   if (out_dtype != MS_BF16 && out_dtype != MS_F32) return MS_BAD_ARG;
-  const GroupedRows grp{rows, tile_expert, (size_t)N * (size_t)K, in_div, out_scatter, act};
+  const GroupedRows grp{rows, tile_expert, (size_t)N * (size_t)K, in_div, out_scatter, act, limit, alpha};
   const bf16* a = (const bf16*)A;
   const bf16* w = (const bf16*)W;
 #define GO(TO, TT) return launch_grouped<TO, TT>(a, (size_t)lda, w, (TO*)out, (size_t)ldo, tiles, N, K, grp, stream)

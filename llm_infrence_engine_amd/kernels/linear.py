@@ -130,6 +130,25 @@ def linear_residual(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tenso
     return linear(a, w, bias)
 
 
+def linear_act(a: torch.Tensor, w: torch.Tensor, epilogue: int, numbers: Optional[torch.Tensor] = None,
+               limit: float = 0.0, alpha: float = 0.0) -> Optional[torch.Tensor]:
+    """A product whose activation is its epilogue (``ops.EPI_RELU2``; ``ops.EPI_CLAMPED`` over interleaved gate and up rows, with
+    its ``limit`` and ``alpha`` also as a float tensor ``numbers`` on the device), where a kernel has it and is the faster way
+    there; None: the caller multiplies and activates in two steps."""
+    if a.dtype != torch.bfloat16:
+        return None
+    try:
+        if ops.skinny_ok(a, w):
+            if epilogue == ops.EPI_RELU2 and ops.splits_columns(a, w):
+                return None
+            return ops.gemm_skinny(a, w, numbers, epilogue)
+        if a.shape[0] > ops.SKINNY_MAX_ROWS and ops.gemm_tiled_pays(a, w):
+            return ops.gemm_tiled(a, w, epilogue, limit, alpha)
+    except ops.UnsupportedShape:
+        _fell_back(a.shape[0], w.shape[0], w.shape[1], "product + activation")
+    return None
+
+
 def linear_swiglu(a: torch.Tensor, w_gate_up: torch.Tensor) -> torch.Tensor:
     """silu(a @ gate.T) * (a @ up.T) for ``w_gate_up`` = interleave_rows(gate, up): [M, I].  ``a`` may be a
     ``LazyNorm``."""

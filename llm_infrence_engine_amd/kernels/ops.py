@@ -43,7 +43,7 @@ _SIGNATURES = {
     "ms_gemm_panel_splitk_parts": [_c_int, _c_int, _c_int],
     "ms_gemm_panel_splitk": [_c_ptr, _c_ll, _c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int,
                              _c_ptr, _c_int, _c_ptr],
-    "ms_gemm_tiled": [_c_ptr, _c_ll, _c_ptr, _c_ll, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+    "ms_gemm_tiled": [_c_ptr, _c_ll, _c_ptr, _c_ll, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_float, _c_float, _c_ptr],
     "ms_gemm_tiled_force": [_c_int],
     "ms_gemm_tiled_force_xcd_split": [_c_int],
     "ms_gemm_tiled_pays": [_c_int, _c_int, _c_int],
@@ -140,7 +140,7 @@ _SIGNATURES = {
     "ms_moe_align": [_c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr],
     "ms_grouped_gemm_mfma_ok": [_c_int, _c_ll, _c_ll, _c_int, _c_int, _c_int],
     "ms_grouped_gemm": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int,
-                        _c_int, _c_int, _c_int, _c_ptr],
+                        _c_int, _c_float, _c_float, _c_int, _c_int, _c_ptr],
     "ms_moe_combine": [_c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_int, _c_ptr, _c_ll, _c_ptr, _c_int, _c_int, _c_int,
                        _c_int, _c_int, _c_ptr],
 }
@@ -473,6 +473,8 @@ def gemm_generic(a: torch.Tensor, w: torch.Tensor, out: torch.Tensor, bias: Opti
 SKINNY_MAX_ROWS = 64
 EPI_STORE, EPI_SWIGLU, EPI_RESIDUAL = 0, 1, 3
 EPI_GEGLU = 4      # as EPI_SWIGLU with the tanh form of the gelu (the tiled product alone has it)
+EPI_RELU2 = 5      # max(product (+ bias), 0)^2
+EPI_CLAMPED = 6    # as EPI_SWIGLU with the clamped gate: min(g, limit) sigmoid(alpha ..) (clamp(u, -limit, limit) + 1)
 
 
 def skinny_ok(a: torch.Tensor, w: torch.Tensor) -> bool:
@@ -487,7 +489,8 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
                 split_columns: bool = True) -> torch.Tensor:
     """a [M <= 64, K] @ w [N, K].T on the matrix cores, bfloat16 in.  Epilogues: EPI_STORE -> [M, N] (+ bias);
     EPI_SWIGLU -> [M, N / 2] = silu(even rows' products) * odd rows' products; EPI_RESIDUAL -> ``residual``
-    (float [M, N]) += product + bias, in place."""
+    (float [M, N]) += product + bias, in place; EPI_RELU2 -> [M, N] = max(product + bias, 0)^2; EPI_CLAMPED -> as EPI_SWIGLU with
+    the clamped gate, whose two numbers (limit, alpha) are ``bias``, a float tensor on the device."""
     _check(a, "a", torch.bfloat16, contiguous=False)
     _check(w, "w", torch.bfloat16)
     if a.dim() != 2 or w.dim() != 2 or a.shape[1] != w.shape[1]:
@@ -497,14 +500,18 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
                          f"and 16-byte aligned rows; got a {list(a.shape)} strides {a.stride()}")
     M, K = a.shape
     N = w.shape[0]
+    gated = epilogue in (EPI_SWIGLU, EPI_CLAMPED)
     if bias is not None:
-        _check(bias, "bias", torch.float32, (N,))
-    if epilogue == EPI_STORE:
+        _check(bias, "bias", torch.float32, (2,) if epilogue == EPI_CLAMPED else (N,))
+    if epilogue in (EPI_STORE, EPI_RELU2):
+        if epilogue == EPI_RELU2:
+            out_dtype = torch.bfloat16
         out = torch.empty((M, N), dtype=out_dtype, device=a.device)
         ldo = N
-    elif epilogue == EPI_SWIGLU:
-        if N % 2 or bias is not None:
-            raise ValueError("the gated epilogue needs an even number of weight rows and no bias")
+    elif gated:
+        if N % 2 or (bias is None) != (epilogue == EPI_SWIGLU):
+            raise ValueError("a gated epilogue needs an even number of weight rows; EPI_SWIGLU takes no bias, EPI_CLAMPED its two "
+                             "numbers")
         out, ldo, out_dtype = torch.empty((M, N // 2), dtype=torch.bfloat16, device=a.device), N // 2, torch.bfloat16
     elif epilogue == EPI_RESIDUAL:
         _check(residual, "residual", torch.float32, (M, N))
@@ -512,7 +519,7 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
     else:
         raise ValueError(f"unknown epilogue {epilogue}")
     lda = a.stride(0) if M > 1 else K
-    if epilogue != EPI_SWIGLU and split_columns:
+    if not gated and epilogue != EPI_RELU2 and split_columns:
         # long rows against few of them (a down projection): the columns are split over blocks too, and the
         # partial sums are added up in a fixed order by a second kernel
         parts = _get("ms_gemm_panel_splitk_parts")(M, N, K)
@@ -524,6 +531,11 @@ def gemm_skinny(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor] =
     _call("ms_gemm_skinny", a.data_ptr(), lda, w.data_ptr(), K, _ptr(bias), out.data_ptr(), ldo,
           M, N, K, epilogue, _code(out_dtype), _stream())
     return out
+
+
+def splits_columns(a: torch.Tensor, w: torch.Tensor) -> bool:
+    """Whether ``gemm_skinny`` spreads the columns of this product over blocks (its sums then pass a second kernel)."""
+    return _get("ms_gemm_panel_splitk_parts")(a.shape[0], w.shape[0], w.shape[1]) > 1
 
 
 def gemm_tiled_pays(a: torch.Tensor, w: torch.Tensor) -> bool:
@@ -541,18 +553,21 @@ def gemm_tiled_plain_pays(a: torch.Tensor, w: torch.Tensor) -> bool:
             and bool(_get("ms_gemm_tiled_plain_pays")(a.shape[0], w.shape[0], a.shape[1])))
 
 
-def gemm_tiled(a: torch.Tensor, w: torch.Tensor, epilogue: int = EPI_STORE) -> torch.Tensor:
+def gemm_tiled(a: torch.Tensor, w: torch.Tensor, epilogue: int = EPI_STORE, limit: float = 0.0, alpha: float = 0.0) -> torch.Tensor:
     """a [M, K] @ w [N, K].T for many rows on the matrix cores, bfloat16 in and out: EPI_STORE -> [M, N];
     EPI_SWIGLU over interleaved rows of w (2j: gate j, 2j + 1: up j) -> [M, N / 2], the product itself never
-    written; EPI_GEGLU: the same with gelu_tanh(gate) for silu(gate).  K a multiple of 64 (else ``UnsupportedShape``)."""
+    written; EPI_GEGLU: the same with gelu_tanh(gate) for silu(gate); EPI_CLAMPED: the same with the clamped gate (``limit``,
+    ``alpha``); EPI_RELU2 -> [M, N] = max(product, 0)^2.  K a multiple of 64 (else ``UnsupportedShape``)."""
     _check(a, "a", torch.bfloat16)
     _check(w, "w", torch.bfloat16, (None, a.shape[1]))
-    if epilogue not in (EPI_STORE, EPI_SWIGLU, EPI_GEGLU):
-        raise ValueError("the tiled product stores its result or the gated activation of it")
+    gated = epilogue in (EPI_SWIGLU, EPI_GEGLU, EPI_CLAMPED)
+    if not gated and epilogue not in (EPI_STORE, EPI_RELU2):
+        raise ValueError("the tiled product stores its result or an activation of it")
     M, K = a.shape
     N = w.shape[0]
-    out = torch.empty((M, N // 2 if epilogue in (EPI_SWIGLU, EPI_GEGLU) else N), dtype=torch.bfloat16, device=a.device)
-    _call("ms_gemm_tiled", a.data_ptr(), K, w.data_ptr(), K, out.data_ptr(), out.shape[1], M, N, K, epilogue, _stream())
+    out = torch.empty((M, N // 2 if gated else N), dtype=torch.bfloat16, device=a.device)
+    _call("ms_gemm_tiled", a.data_ptr(), K, w.data_ptr(), K, out.data_ptr(), out.shape[1], M, N, K, epilogue, float(limit),
+          float(alpha), _stream())
     return out
 
 
@@ -1295,7 +1310,8 @@ def latent_kv_store(kv: torch.Tensor, norm_weight: torch.Tensor, eps: float, pos
     latent_prepare(positions, inv_freq, gain, half, kv=(kv, norm_weight, eps, slot_mapping, c_pages, r_pages, ct_pages))
 
 
-LATENT_SPLIT_BLOCKS = 512     # blocks a step of single tokens aims to put on the chip
+LATENT_SPLIT_BLOCKS = 256     # blocks a step of single tokens aims to put on the chip: one to a CU (64 requests, 28 heads, 540
+# keys of 512 + 64: 47 us unsplit, 39 in 2, 51 in 4; 8 requests: 40, 29, 24 and 21 in 8; at 4,096 keys 222 and 38 in 16)
 
 
 def latent_splits(n_requests: int, heads: int, max_q_len: int, max_context_len: int, window: Optional[int]) -> int:
@@ -1564,10 +1580,12 @@ def moe_align(ids: torch.Tensor, n_experts: int, tile: Optional[int] = None):
 
 
 def grouped_gemm(a: torch.Tensor, w: torch.Tensor, rows: torch.Tensor, tile_expert: torch.Tensor, out: torch.Tensor,
-                 gather_div: int = 0, scatter: bool = False, act: Optional[str] = None) -> torch.Tensor:
+                 gather_div: int = 0, scatter: bool = False, act: Optional[str] = None, limit: float = 0.0,
+                 alpha: float = 0.0) -> torch.Tensor:
     """For every tile with an expert e and every row of it (flat position p, item = rows[p] >= 0):
     out[item if scatter else p] = act(a[item // gather_div if gather_div else p] @ w[e].T); w [experts, n_out, K]; float
-    accumulation in the order of K.  ``act``: None or "gelu".  The tiles' size is read off ``rows`` and ``tile_expert``
+    accumulation in the order of K.  ``act``: None, "gelu", or "clamped_glu" (``limit``, ``alpha``) over interleaved gate and up
+    rows of w, out [., n_out / 2], for products that run on the matrix cores (else ``UnsupportedShape``).  The tiles' size is read off ``rows`` and ``tile_expert``
     (``moe_align``'s); bfloat16 with K a multiple of 32 runs on the matrix cores (the widest tiles: a multiple of 64),
     everything else on the vector ALUs (tiles of ``moe_tile_rows()`` rows only)."""
     _check(w, "w", a.dtype)
@@ -1575,7 +1593,9 @@ def grouped_gemm(a: torch.Tensor, w: torch.Tensor, rows: torch.Tensor, tile_expe
         raise ValueError("w must be [experts, out features, in features]")
     E, n_out, K = w.shape
     a_stride = _rows2d(a, "a", None, K)
-    o_stride = _rows2d(out, "out", None, n_out)
+    if act == "clamped_glu" and (n_out % 2 or out.dtype != torch.bfloat16):
+        raise UnsupportedShape("the gated epilogue of the grouped product is for bfloat16 results of gate and up in pairs")
+    o_stride = _rows2d(out, "out", None, n_out // 2 if act == "clamped_glu" else n_out)
     _check(tile_expert, "tile_expert", torch.int32)
     tiles = tile_expert.numel()
     _check(rows, "rows", torch.int32)
@@ -1587,10 +1607,11 @@ def grouped_gemm(a: torch.Tensor, w: torch.Tensor, rows: torch.Tensor, tile_expe
         raise ValueError("a must hold a row for every row of every tile")
     if not scatter and out.shape[0] < tiles * tile:
         raise ValueError("out must hold a row for every row of every tile")
-    if act not in (None, "gelu"):
+    if act not in (None, "gelu", "clamped_glu"):
         raise ValueError(f"no activation {act!r} here")
     _call("ms_grouped_gemm", a.data_ptr(), a_stride, w.data_ptr(), rows.data_ptr(), tile_expert.data_ptr(), out.data_ptr(),
-          o_stride, tiles, tile, n_out, K, int(gather_div), int(scatter), int(act == "gelu"), _code(a.dtype),
+          o_stride, tiles, tile, n_out, K, int(gather_div), int(scatter), {None: 0, "gelu": 1, "clamped_glu": 2}[act],
+          float(limit), float(alpha), _code(a.dtype),
           _code(out.dtype), _stream())
     return out
 

@@ -102,7 +102,16 @@ class RoutedExperts(FeedForward):
         logits = linear.linear(h, self.w_router, out_dtype=torch.float32)
         ids, weights = ops.moe_route(logits, self.correction, self.top, E + self.identity, self.scores, self.groups, self.normalise)
         rows, tile_expert = ops.moe_align(ids, E, ops.moe_tile_choice(ids.numel(), E, (W, self.expert_ff), h.dtype))
-        if self.gated:
+        mid = None
+        if self.activation == "clamped_glu" and h.dtype == torch.bfloat16 and W % 32 == 0:
+            try:            # on the matrix cores the gate is the product's epilogue
+                mid = ops.grouped_gemm(h, self.w_up, rows, tile_expert, self.rt.empty(rows.numel(), self.expert_ff),
+                                       gather_div=self.top, act="clamped_glu", limit=self.limit, alpha=self.alpha)
+            except ops.UnsupportedShape:
+                mid = None
+        if mid is not None:
+            pass
+        elif self.gated:
             gu = ops.grouped_gemm(h, self.w_up, rows, tile_expert, self.rt.empty(rows.numel(), 2 * self.expert_ff),
                                   gather_div=self.top)
             mid = self.rt.empty(rows.numel(), self.expert_ff)

@@ -60,6 +60,9 @@ class DenseAct(FeedForward):
         return self.forward_residual(h, ctx, None)
 
     def forward_residual(self, h, ctx, x):
+        u = linear.linear_act(h, self.w_up, ops.EPI_RELU2) if self.activation == "relu2" else None
+        if u is not None:
+            return linear.linear_residual(u, self.w_down, None, x)
         u = linear.linear(h, self.w_up)
         if self.activation == "xielu":
             u = ops.xielu(u, self.act, torch.empty_like(u))
@@ -87,10 +90,13 @@ class ClampedGLU(FeedForward):
         g, u, d = (get(s) for s in self.tensor_specs())
         self.w_gate_up = linear.interleave_rows(g, u)
         self.w_down = linear.prepare_weight(d)
+        self.numbers = torch.tensor([self.limit, self.alpha], dtype=torch.float32, device=rt.device)
 
     def forward(self, h, ctx):
-        gu = linear.linear(h, self.w_gate_up)
-        act = ops.clamped_glu(gu, self.rt.empty(gu.shape[0], self.intermediate_size), self.limit, self.alpha)
+        act = linear.linear_act(h, self.w_gate_up, ops.EPI_CLAMPED, self.numbers, self.limit, self.alpha)
+        if act is None:
+            gu = linear.linear(h, self.w_gate_up)
+            act = ops.clamped_glu(gu, self.rt.empty(gu.shape[0], self.intermediate_size), self.limit, self.alpha)
         return linear.linear(act, self.w_down)
 
 
