@@ -1310,8 +1310,9 @@ def latent_kv_store(kv: torch.Tensor, norm_weight: torch.Tensor, eps: float, pos
     latent_prepare(positions, inv_freq, gain, half, kv=(kv, norm_weight, eps, slot_mapping, c_pages, r_pages, ct_pages))
 
 
-LATENT_SPLIT_BLOCKS = 256     # blocks a step of single tokens aims to put on the chip: one to a CU (64 requests, 28 heads, 540
-# keys of 512 + 64: 47 us unsplit, 39 in 2, 51 in 4; 8 requests: 40, 29, 24 and 21 in 8; at 4,096 keys 222 and 38 in 16)
+# Blocks a step of single tokens aims to put on the chip: one to a CU.  (64 requests, 28 heads, 540 keys of 512 + 64: 47 us
+# unsplit, 39 in 2, 51 in 4; 8 requests: 40, 29 in 2, 24 in 4, 21 in 8; 8 requests of 4,096 keys: 222, 38 in 16.)
+LATENT_SPLIT_BLOCKS = 256
 
 
 def latent_splits(n_requests: int, heads: int, max_q_len: int, max_context_len: int, window: Optional[int]) -> int:
