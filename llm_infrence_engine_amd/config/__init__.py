@@ -8,8 +8,10 @@ from .gidurax import GiduraxConfig
 from .kuvazen import KuvazenConfig
 from .silizen import SilizenConfig
 from .gositar import GositarConfig
+from .kisusun import KisusunConfig
 from .presets import PRESETS, preset
 
 __all__ = ["EngineConfig", "ConfigError", "build_spec", "config_class", "config_from_dict",
            "known_architectures", "load_config", "register_architecture", "LayerSpec", "ModelSpec",
-           "PartSpec", "Run", "layer", "Qwen2Config", "GemadraConfig", "GiduraxConfig", "KuvazenConfig", "SilizenConfig", "GositarConfig", "PRESETS", "preset"]
+           "PartSpec", "Run", "layer", "Qwen2Config", "GemadraConfig", "GiduraxConfig", "KuvazenConfig", "SilizenConfig", "GositarConfig",
+           "KisusunConfig", "PRESETS", "preset"]

@@ -1,5 +1,5 @@
 """Named config.json contents for the random-weights mode: the shapes the published Qwen2.5 checkpoints
-have, the two tiny ones the tests use and two Gemadra, two Gidurax, two Kuvazen, two Silizen and two Gositar shapes of the same widths, so that ``--random-config 0.5b``
+have, the two tiny ones the tests use and two Gemadra, two Gidurax, two Kuvazen, two Silizen, two Gositar and two Kisusun shapes of the same widths, so that ``--random-config 0.5b``
 needs no file.  These are data
 of the kind a config.json holds; no part or kernel reads them.
 """
@@ -144,6 +144,30 @@ PRESETS["gositar-0.5b"] = _gositar(
 PRESETS["gositar-7b"] = _gositar(
     3584, 28416, 28, 4, {"heads": 28, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 192 ** -0.5,
                          "rot": {"base": 10000.0, "dims": 64, "scaling": _YARN}}, (6336, 16, 2, 4, 2, 6272), vocab=152064)
+
+
+def _kisusun(width, ff, layers, attention, window, experts, vocab=151936):
+    """``layers`` layers, every second feed-forward routed (``experts``: (expert ff, experts, top, groups, kept groups, shared
+    ff)); a window in every layer but each fourth one."""
+    import copy
+
+    ef, n, top, count, keep, shared = experts
+    routed = {"kind": "moe", "expert": {"ff": ef, "limit": 7.0}, "router": {"experts": n, "top": top, "scale": 1.0,
+              "groups": {"count": count, "keep": keep}}, "shared": {"ff": shared, "limit": 7.0}}
+    mixer = dict(attention, softcap=50.0, v_mix=True, rot={"base": 1000000.0, "dims": attention["dim"] // 2, "scaling": {"factor": 8.0}})
+    return {"architecture": "Kisusun", "vocab": vocab, "width": width, "norm": {"eps": 1e-6},
+            "embedding": {"scale": float(width) ** 0.5}, "logit_scale": 1.0,
+            "layers": [{"type": "attention", "mixer": copy.deepcopy(dict(mixer, mask={"size": window}) if i % 4 != 3 else mixer),
+                        "mlp": copy.deepcopy(routed) if i % 2 else {"kind": "dense", "ff": ff}} for i in range(layers)]}
+
+
+# Kisusun at the same widths: attention of the Qwen2 shapes' heads, a window of 1,024 tokens, gated dense feed-forwards of the
+# Qwen2 shapes' size, routed ones of Gositar's
+PRESETS["kisusun-0.5b"] = _kisusun(
+    896, 4864, 24, {"heads": 14, "kv_heads": 2, "dim": 64, "vdim": 64, "scale": 64 ** -0.5}, 1024, (1600, 16, 2, 4, 2, 1664))
+PRESETS["kisusun-7b"] = _kisusun(
+    3584, 18944, 28, {"heads": 28, "kv_heads": 4, "dim": 128, "vdim": 128, "scale": 128 ** -0.5}, 1024,
+    (6336, 16, 2, 4, 2, 6272), vocab=152064)
 
 
 def preset(name: str) -> dict:

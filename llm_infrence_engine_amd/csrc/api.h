@@ -108,25 +108,25 @@ int ms_paged_attention_generic(const void* q, long long q_stride, const void* k_
                                void* out, long long out_stride, int n_tokens, int num_heads, int num_kv_heads,
                                int head_dim, int value_dim, int page_size, long long num_pages, float scale, int window,
                                int v_transposed, const float* sink, float softcap, const float* slopes, const void* gate,
-                               long long gate_stride, float out_scale, int dtype, hipStream_t stream);
+                               long long gate_stride, int gate_width, float out_scale, int dtype, hipStream_t stream);
 
-int ms_attention_mfma_supported(int head_dim, int page_size);
+int ms_attention_mfma_supported(int head_dim, int value_dim, int page_size);
 
 int ms_paged_attention_mfma(const void* q, long long q_stride, const void* k_pages, const void* vt_pages,
                             const int* block_table, int table_stride, const int* table_rows, const int* q_start,
                             const int* context_lens, void* out, long long out_stride, int n_requests, int n_tokens,
-                            int max_q_len, int num_heads, int num_kv_heads, int head_dim, int page_size, float scale,
+                            int max_q_len, int num_heads, int num_kv_heads, int head_dim, int value_dim, int page_size, float scale,
                             int window, const float* sink, float softcap, const float* slopes, const void* gate,
-                            long long gate_stride, float out_scale, hipStream_t stream);
+                            long long gate_stride, int gate_width, float out_scale, hipStream_t stream);
 
 int ms_paged_attention_mfma_decode(const void* q, long long q_stride, const void* k_pages, const void* vt_pages,
                                    const int* block_table, int table_stride, const int* table_rows,
                                    const int* q_start, const int* context_lens, void* out, long long out_stride,
                                    void* part_o,
                                    void* part_ml, int n_requests, int num_heads, int num_kv_heads, int head_dim,
-                                   int page_size, float scale, int window, int min_blocks, int n_splits,
+                                   int value_dim, int page_size, float scale, int window, int min_blocks, int n_splits,
                                    const float* sink, float softcap, const float* slopes, const void* gate,
-                                   long long gate_stride, float out_scale, hipStream_t stream);
+                                   long long gate_stride, int gate_width, float out_scale, hipStream_t stream);
 
 int ms_argmax(const float* logits, long long ld, int n_rows, int vocab, float* scratch_val, int* scratch_idx,
               int n_chunks, int* out, hipStream_t stream);
@@ -217,10 +217,11 @@ int ms_latent_attention_mfma(const void* q, long long q_tok, long long q_head, c
 
 // ---- layers that normalise a sublayer's output before it joins the residual stream (csrc/residual_norm.hip)
 // x += w_post * rms_norm(y); then, if out is not null, out = w_next * rms_norm(x).  y [n, hidden] in y_dtype (rows y_stride
-// apart), x float [n, hidden], out in out_dtype.
-int ms_rms_norm_add(const void* y, long long y_stride, int y_dtype, const float* w_post, float eps_post, float* x,
-                    const float* w_next, float eps_next, void* out, int out_dtype, int n_rows, int hidden,
-                    hipStream_t stream);
+// apart), x float [n, hidden], out in out_dtype.  w_next null: out = x rounded.  parts not null: y (then optional)
+// + sum_j part_weights[n, j] parts[n top + j] stands for y.  w_post null: x is left as it is (no y, no parts).
+int ms_rms_norm_add(const void* y, long long y_stride, int y_dtype, const float* parts, const float* part_weights, int top,
+                    const float* w_post, float eps_post, float* x, const float* w_next, float eps_next,
+                    void* out, int out_dtype, int n_rows, int hidden, hipStream_t stream);
 // x[n, :] += kept[n, :] (if not null) + vec[:] (if not null)
 int ms_add_rows(float* x, const float* kept, const float* vec, int n_rows, int hidden, hipStream_t stream);
 
@@ -232,6 +233,13 @@ int ms_qk_norm_store(void* qkv, long long stride, const float* q_weight, const f
                      const int* positions, float coef, int every, const int* slots, void* k_pages, void* v_pages,
                      int n_tokens, int num_heads, int num_kv_heads, int head_dim, int value_dim, int page_size,
                      int v_transposed, int unit_norm, const float* inv_freq, int rot_dim, int dtype, hipStream_t stream);
+// all q heads (all k heads) of a token through one RMS norm with a weight per entry of the projection, the rotation as above,
+// then k and the values, blended with `first` by *lambda where given, into the pages
+int ms_qk_span_norm_store(void* qkv, long long stride, const float* q_weight, const float* k_weight, float eps,
+                          const int* positions, const float* inv_freq, int rot_dim, const void* first, long long first_stride,
+                          const float* lambda, const int* slots, void* k_pages, void* v_pages, int n_tokens, int num_heads,
+                          int num_kv_heads, int head_dim, int value_dim, int page_size, int v_transposed, int dtype,
+                          hipStream_t stream);
 
 // ---- the selective scan of a state-space mixer (csrc/scan.hip)
 int ms_selective_scan(const void* x, long long x_stride, const float* dt_in, const float* dt_bias, const float* A,
@@ -246,7 +254,8 @@ int ms_relu2(const void* x, void* out, long long total, int dtype, hipStream_t s
 // score + correction: ids / weights [n, top]; groups > 0: among the outputs of the `keep` best of so many equal groups of
 // neighbours; normalise: weights divided by their sum
 int ms_moe_route(const float* logits, long long ld, const float* correction, int n_tokens, int n_out, int top, int* ids,
-                 float* weights, int sigmoid_scores, int groups, int keep, int normalise, hipStream_t stream);
+                 float* weights, int sigmoid_scores, int groups, int keep, int group_top, int normalise, float weight_scale,
+                 hipStream_t stream);
 int ms_moe_tile_rows();
 int ms_moe_wide_tile_rows();
 // rows [tiles * tile] and tile_expert [tiles] from ids [n_items]; ids >= n_experts take no row; tile: ms_moe_tile_rows()

@@ -7,7 +7,8 @@
 // n_live_tokens (null: all): a device int; tokens from that index on belong to no request and are skipped.
 // `softcap` > 0: a score s (already scaled) becomes softcap * tanh(s / softcap).  `slopes` (may be null): one number per
 // query head; slope * (distance of the key from the query) is taken off the score, after the cap.  `gate` (may be null):
-// one number per token and query head, the head's result is multiplied by sigmoid(gate); `out_scale` multiplies all.
+// `gate_width` numbers per token and query head, 1 (the head's result is multiplied by sigmoid(gate)) or the value size (every
+// entry by a sigmoid of its own); `out_scale` multiplies all.
 // This is the attention of the 32-bit path and the any-shape fallback of the bfloat16 path.
 #include "common.h"
 #include "api.h"
@@ -26,7 +27,7 @@ paged_attention_generic_kernel(const T* __restrict__ q, size_t q_stride, const T
                                T* __restrict__ out, size_t out_stride, int n_tokens, int nh, int nkv, int d, int dv,
                                int page_size, float scale, int window, int v_transposed,
                                const float* __restrict__ sink, float softcap, const float* __restrict__ slopes,
-                               const T* __restrict__ gate, size_t gate_stride, float out_scale) {
+                               const T* __restrict__ gate, size_t gate_stride, int gate_width, float out_scale) {
   __shared__ float qs[WAVES][MAX_D];
   const int lane = threadIdx.x & (MS_WAVE - 1), wave = threadIdx.x / MS_WAVE;
   const long long item = (long long)blockIdx.x * WAVES + wave;
@@ -101,11 +102,12 @@ paged_attention_generic_kernel(const T* __restrict__ q, size_t q_stride, const T
   T* op = out + (size_t)n * out_stride + (size_t)h * dv;
   if (sink) l += expf(sink[h] - m);   // m is finite: a token always sees its own key
   float inv = out_scale / l;
-  if (gate) inv /= 1.0f + expf(-to_float(gate[(size_t)n * gate_stride + h]));
+  const T* gp = gate ? gate + (size_t)n * gate_stride + (size_t)h * gate_width : nullptr;
+  if (gate && gate_width == 1) { inv /= 1.0f + expf(-to_float(*gp)); gp = nullptr; }
 #pragma unroll
   for (int c = 0; c < MAX_D / MS_WAVE; ++c) {
     const int i = lane + c * MS_WAVE;
-    if (i < dv) op[i] = from_float<T>(acc[c] * inv);
+    if (i < dv) op[i] = from_float<T>(gp ? acc[c] * inv / (1.0f + expf(-to_float(gp[i]))) : acc[c] * inv);
   }
 }
 
@@ -118,15 +120,17 @@ extern "C" int ms_paged_attention_generic(const void* q, long long q_stride, con
                                           int num_heads, int num_kv_heads, int head_dim, int value_dim, int page_size,
                                           long long num_pages, float scale, int window, int v_transposed,
                                           const float* sink, float softcap, const float* slopes, const void* gate,
-                                          long long gate_stride, float out_scale, int dtype, hipStream_t stream) {
+                                          long long gate_stride, int gate_width, float out_scale, int dtype,
+                                          hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
   if (num_heads <= 0 || num_kv_heads <= 0 || num_heads % num_kv_heads || page_size <= 0 || table_stride <= 0)
     return MS_BAD_ARG;
   if (head_dim <= 0 || head_dim > MAX_D || value_dim <= 0 || value_dim > MAX_D) return MS_UNSUPPORTED;
+  if (gate != nullptr && gate_width != 1 && gate_width != value_dim) return MS_BAD_ARG;
   if (num_pages * num_kv_heads * page_size >= (1ll << 31)) return MS_UNSUPPORTED;  // row index is an int
   const long long items = (long long)n_tokens * num_heads;
   dim3 grid((unsigned)((items + WAVES - 1) / WAVES)), block(WAVES * MS_WAVE);
-#define LAUNCH(T) paged_attention_generic_kernel<T><<<grid, block, 0, stream>>>((const T*)q, (size_t)q_stride, (const T*)k_pages, (const T*)v_pages, block_table, table_stride, table_rows, n_live_tokens, token_req, positions, (T*)out, (size_t)out_stride, n_tokens, num_heads, num_kv_heads, head_dim, value_dim, page_size, scale, window, v_transposed, sink, softcap, slopes, (const T*)gate, (size_t)gate_stride, out_scale)
+#define LAUNCH(T) paged_attention_generic_kernel<T><<<grid, block, 0, stream>>>((const T*)q, (size_t)q_stride, (const T*)k_pages, (const T*)v_pages, block_table, table_stride, table_rows, n_live_tokens, token_req, positions, (T*)out, (size_t)out_stride, n_tokens, num_heads, num_kv_heads, head_dim, value_dim, page_size, scale, window, v_transposed, sink, softcap, slopes, (const T*)gate, (size_t)gate_stride, gate_width, out_scale)
   if (dtype == MS_F32) LAUNCH(float);
   else if (dtype == MS_BF16) LAUNCH(bf16);
   else return MS_BAD_ARG;

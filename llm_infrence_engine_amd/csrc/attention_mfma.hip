@@ -39,6 +39,10 @@ typedef __attribute__((ext_vector_type(4))) float f32x4;
 
 __device__ __forceinline__ float fast_exp2(float x) { return __builtin_amdgcn_exp2f(x); }
 
+__device__ __forceinline__ float fast_sigmoid(float x) {
+  return __builtin_amdgcn_rcpf(1.0f + fast_exp2(-1.4426950408889634f * x));
+}
+
 constexpr float REF_SLACK = 8.0f;   // log2 units by which a column's maximum may run ahead of its reference
 
 template <int D>
@@ -70,15 +74,18 @@ __device__ __forceinline__ void pages_of(const int* __restrict__ table, int base
 
 // Where the two 16-key halves of a block start inside their page's part of one kv head: uniform values.
 struct BlockPlace {
-  size_t head[2];   // element offset of (page, kv head) in either pool
+  size_t head[2];   // element offset of (page, kv head) in the keys' pool
+  size_t vhead[2];  // and in the values' pool (the same unless values are narrower than keys)
   int off[2];       // first key inside the page
 };
 
-__device__ __forceinline__ BlockPlace place_of(const int* pages, int base, int g, int nkv, PageGeom pg, int D) {
+__device__ __forceinline__ BlockPlace place_of(const int* pages, int base, int g, int nkv, PageGeom pg, int D,
+                                               int DV) {
   BlockPlace bp;
 #pragma unroll
   for (int u = 0; u < 2; ++u) {
     bp.head[u] = ((size_t)pages[u] * nkv + g) * pg.size * D;
+    bp.vhead[u] = DV == D ? bp.head[u] : ((size_t)pages[u] * nkv + g) * pg.size * DV;
     bp.off[u] = pg.offset(base + u * 16);
   }
   return bp;
@@ -96,15 +103,16 @@ __device__ __forceinline__ void load_keys(KeyBlock<D>& b, const bf16* __restrict
   }
 }
 
-template <int CT>
+template <int CT, bool NARROW>
 __device__ __forceinline__ void load_values(ValueBlock<CT>& b, const bf16* __restrict__ vt_pages,
-                                            const BlockPlace& bp, PageGeom pg, int dim0, int lane) {
+                                            const BlockPlace& bp, PageGeom pg, int dim0, int lane, int live) {
   const int v_lane = (dim0 + (lane & 15)) * pg.size + (lane >> 4) * 4;   // this lane's dim and keys inside a tile
 #pragma unroll
   for (int u = 0; u < 2; ++u) {
-    const bf16* vp = vt_pages + bp.head[u] + bp.off[u];
+    const bf16* vp = vt_pages + bp.vhead[u] + bp.off[u];
 #pragma unroll
-    for (int c = 0; c < CT; ++c) b.v[c][u] = *reinterpret_cast<const bf16x4*>((vp + c * 16 * pg.size) + v_lane);
+    for (int c = 0; c < CT; ++c)
+      if (!NARROW || c < live) b.v[c][u] = *reinterpret_cast<const bf16x4*>((vp + c * 16 * pg.size) + v_lane);
   }
 }
 
@@ -116,16 +124,18 @@ __device__ __forceinline__ void load_values(ValueBlock<CT>& b, const bf16* __res
 // shortens the longest chain without a second kernel; the blocks write disjoint dims and share nothing.
 // EXTRA: the scores are changed on their way into the softmax: a scaled score x becomes cap * tanh(x / cap) (cap > 0),
 // then slope * (the key's distance from the query) is taken off it, one slope per query head; at the end every head's
-// result is multiplied by out_scale and by the sigmoid of a gate, one number per token and head.  Such scores are kept
+// result is multiplied by out_scale and by the sigmoid of a gate, one number per token and head or one per entry.  Such scores are kept
 // in log2 units from the start, and the block's maxima are those of the changed scores.
 struct AttnExtras {
   float scale;               // of the raw scores, natural units
   float cap;                 // 0: no cap
   float exp_arg;             // 2 log2(e) / cap: tanh(x / cap) = 1 - 2 / (2^(x exp_arg) + 1)
   const float* slopes;       // [nh] or null
-  const bf16* gate;          // [N, >= nh] or null
+  const bf16* gate;          // [N, >= nh * gate_width] or null
   size_t gate_stride;
+  int gate_width;            // 1, or the value size
   float out_scale;
+  int value_dim;             // the value size (NARROW variants: below the key size)
 };
 
 // The variants that change their scores need more registers than two wide tiles to a SIMD leave: a wide tile of theirs
@@ -136,7 +146,9 @@ constexpr bool extra_variant() {
   return !(NT == 1 && WAVES == 16) && !(D == 128 && NT == 1 && WAVES == 8 && VS == 1) && !(NT > 1 && WAVES == 8);
 }
 
-template <int D, int NT, int WAVES, bool SPLIT, int VS, bool SINK, bool EXTRA = false>
+// NARROW: values have fewer dims than keys (a multiple of 16); the tiles of 16 dims past them are neither read nor
+// multiplied, which a branch that is the same for the whole launch decides.
+template <int D, int NT, int WAVES, bool SPLIT, int VS, bool SINK, bool EXTRA = false, bool NARROW = false>
 __global__ void __launch_bounds__(WAVES * MS_WAVE, (NT > 1 && !EXTRA ? 2 : 1))
 attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* __restrict__ k_pages,
                       const bf16* __restrict__ vt_pages, const int* __restrict__ block_table, int table_stride,
@@ -151,7 +163,10 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
   __shared__ float sm_m[WAVES][NT][16], sm_l[WAVES][NT][16];
   static_assert(VS == 1 || (NT == 1 && !SPLIT), "only narrow tiles of the general shape share their dims out");
   static_assert((D / 16) % VS == 0, "whole tiles of 16 dims to a block");
+  static_assert(!NARROW || (EXTRA && VS == 1), "narrow values come with the variants that change their scores");
   constexpr int CT = D / 16 / VS;
+  const int DV = NARROW ? ex.value_dim : D;
+  const int live = NARROW ? DV / 16 : CT;     // tiles of 16 value dims
   __shared__ f32x4 sm_o[WAVES > 1 ? WAVES - 1 : 1][CT][NT][MS_WAVE];
   const int lane = threadIdx.x & (MS_WAVE - 1);
   const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / MS_WAVE);   // the same for the whole wave
@@ -319,9 +334,9 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
     } else {
       pages_of(table, base, key_hi, pg, pages);
     }
-    cur_at = place_of(pages, base, g, nkv, pg, D);
+    cur_at = place_of(pages, base, g, nkv, pg, D, DV);
     load_keys<D>(cur_k, k_pages, cur_at, lane);
-    if (VALUES_EARLY) load_values<CT>(cur_v, vt_pages, cur_at, pg, dim0, lane);
+    if (VALUES_EARLY) load_values<CT, NARROW>(cur_v, vt_pages, cur_at, pg, dim0, lane, live);
   }
   // The page ids of a block are asked for one block before its keys are: the keys' loads then go out at the top of
   // an iteration instead of behind a table lookup (8,192 tokens of the 0.5B shape: 235 -> 232 us; 2,048 tokens at
@@ -334,11 +349,11 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
   auto step = [&](int blk, KeyBlock<D>& cur_k, ValueBlock<CT>& cur_v, BlockPlace& cur_at, KeyBlock<D>& nxt_k,
                   ValueBlock<CT>& nxt_v, BlockPlace& nxt_at) __attribute__((always_inline)) {
     const int base = blk * 32;
-    if (!VALUES_EARLY) load_values<CT>(cur_v, vt_pages, cur_at, pg, dim0, lane);
+    if (!VALUES_EARLY) load_values<CT, NARROW>(cur_v, vt_pages, cur_at, pg, dim0, lane, live);
     if (blk + WAVES < blk_end) {
-      nxt_at = place_of(ahead_pages, base + WAVES * 32, g, nkv, pg, D);
+      nxt_at = place_of(ahead_pages, base + WAVES * 32, g, nkv, pg, D, DV);
       load_keys<D>(nxt_k, k_pages, nxt_at, lane);
-      if (VALUES_EARLY) load_values<CT>(nxt_v, vt_pages, nxt_at, pg, dim0, lane);
+      if (VALUES_EARLY) load_values<CT, NARROW>(nxt_v, vt_pages, nxt_at, pg, dim0, lane, live);
       if (blk + 2 * WAVES < blk_end) pages_of(table, base + 2 * WAVES * 32, key_hi, pg, ahead_pages);
     }
 
@@ -378,7 +393,8 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
         for (int i = 0; i < 4; ++i)
           if (base + u * 16 + kq * 4 + i > key_hi) {
 #pragma unroll
-            for (int c = 0; c < CT; ++c) cur_v.v[c][u][i] = (__bf16)0.0f;
+            for (int c = 0; c < CT; ++c)
+              if (!NARROW || c < live) cur_v.v[c][u][i] = (__bf16)0.0f;
           }
     }
 
@@ -456,6 +472,7 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
       if (SUMS_BY_MATRIX) lsum[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, p[t], lsum[t], 0, 0, 0);
 #pragma unroll
       for (int c = 0; c < CT; ++c) {
+        if (NARROW && c >= live) break;
         bf16x8 vv;
 #pragma unroll
         for (int i = 0; i < 4; ++i) { vv[i] = cur_v.v[c][0][i]; vv[4 + i] = cur_v.v[c][1][i]; }
@@ -519,23 +536,32 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
     if (SPLIT) {
       // unnormalised: O, the running maximum (log2 units) and the sum; the combine kernel weighs the splits
       const size_t slot = ((size_t)r * nh + head) * n_splits + bx;
-      float* po = part_o + slot * D + kq * 4;
+      float* po = part_o + slot * DV + kq * 4;
 #pragma unroll
-      for (int c = 0; c < CT; ++c) *reinterpret_cast<f32x4*>(po + c * 16) = o[c][t];
+      for (int c = 0; c < CT; ++c)
+        if (!NARROW || c < live) *reinterpret_cast<f32x4*>(po + c * 16) = o[c][t];
       if (kq == 0) { part_ml[slot * 2] = m[t]; part_ml[slot * 2 + 1] = lt; }
     } else {
       float inv = 1.0f / lt;
       if (EXTRA) {
         inv *= ex.out_scale;
-        if (ex.gate)
-          inv *= __builtin_amdgcn_rcpf(1.0f + fast_exp2(-1.4426950408889634f * __bfloat162float(ex.gate[(size_t)tok * ex.gate_stride + head])));
+        if (ex.gate && ex.gate_width == 1)
+          inv *= fast_sigmoid(__bfloat162float(ex.gate[(size_t)tok * ex.gate_stride + head]));
       }
-      bf16* op = out + (size_t)tok * out_stride + (size_t)head * D + dim0 + kq * 4;
+      const bool by_entry = EXTRA && ex.gate && ex.gate_width != 1;
+      const bf16* gp = by_entry ? ex.gate + (size_t)tok * ex.gate_stride + (size_t)head * DV + dim0 + kq * 4 : nullptr;
+      bf16* op = out + (size_t)tok * out_stride + (size_t)head * DV + dim0 + kq * 4;
 #pragma unroll
       for (int c = 0; c < CT; ++c) {
+        if (NARROW && c >= live) break;
         bf16x4 w;
 #pragma unroll
         for (int i = 0; i < 4; ++i) w[i] = (__bf16)(o[c][t][i] * inv);
+        if (by_entry) {
+          const bf16x4 gv = *reinterpret_cast<const bf16x4*>(gp + c * 16);
+#pragma unroll
+          for (int i = 0; i < 4; ++i) w[i] = (__bf16)(o[c][t][i] * inv * fast_sigmoid((float)gv[i]));
+        }
         *reinterpret_cast<bf16x4*>(op + c * 16) = w;
       }
     }
@@ -551,8 +577,8 @@ template <int D>
 __global__ void __launch_bounds__(D < 64 ? 64 : D)
 attention_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
                          const int* __restrict__ q_start, const int* __restrict__ context_lens,
-                         bf16* __restrict__ out, size_t out_stride, int nh, int window, int min_blocks,
-                         int n_splits, const bf16* __restrict__ gate, size_t gate_stride, float out_scale) {
+                         bf16* __restrict__ out, size_t out_stride, int nh, int dv, int window, int min_blocks,
+                         int n_splits, const bf16* __restrict__ gate, size_t gate_stride, int gate_width, float out_scale) {
   __shared__ float sm_m[COMBINE_MAX_SPLITS], sm_w[COMBINE_MAX_SPLITS];
   const int r = blockIdx.x / nh, h = blockIdx.x % nh;
   if (q_start[r + 1] == q_start[r]) return;   // a row that pads a captured batch: no token, nothing to write
@@ -578,13 +604,16 @@ attention_combine_kernel(const float* __restrict__ part_o, const float* __restri
   float den = 0.f;
   for (int s = 0; s < used; ++s) den += sm_m[s];
   float inv = out_scale / den;
-  if (gate) inv *= 1.0f / (1.0f + expf(-__bfloat162float(gate[(size_t)q_start[r] * gate_stride + h])));
-  bf16* op = out + (size_t)q_start[r] * out_stride + (size_t)h * D;
-  for (int d = t; d < D; d += blockDim.x) {
+  const bf16* gp = gate ? gate + (size_t)q_start[r] * gate_stride + (size_t)h * gate_width : nullptr;
+  if (gate && gate_width == 1) inv *= 1.0f / (1.0f + expf(-__bfloat162float(*gp)));
+  bf16* op = out + (size_t)q_start[r] * out_stride + (size_t)h * dv;
+  for (int d = t; d < dv; d += blockDim.x) {
     float acc = 0.f;
 #pragma unroll 8
-    for (int s = 0; s < used; ++s) acc += sm_w[s] * part_o[(slot0 + s) * D + d];
-    op[d] = __float2bfloat16(acc * inv);
+    for (int s = 0; s < used; ++s) acc += sm_w[s] * part_o[(slot0 + s) * dv + d];
+    acc *= inv;
+    if (gate && gate_width != 1) acc /= 1.0f + expf(-__bfloat162float(gp[d]));
+    op[d] = __float2bfloat16(acc);
   }
 }
 
@@ -614,6 +643,14 @@ int launch_general(const bf16* q, size_t q_stride, const bf16* k, const bf16* vt
   if constexpr (D == 64 && NT == 4) {     // no variant with a sink or changed scores at this shape (its registers are spent)
     if (sink || extras) return MS_UNSUPPORTED;
   } else if (extras) {
+    if (extras->value_dim != D) {
+      if constexpr (VS == 1 && extra_variant<D, NT, WAVES, VS>()) {
+        attention_mfma_kernel<D, NT, WAVES, false, VS, true, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, nullptr, nullptr, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, pair_order, scan, sink, *extras);
+        return ms_launch_status();
+      } else {
+        return MS_UNSUPPORTED;
+      }
+    }
     if constexpr (extra_variant<D, NT, WAVES, VS>()) {
       attention_mfma_kernel<D, NT, WAVES, false, VS, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, nullptr, nullptr, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, pair_order, scan, sink, *extras);
       return ms_launch_status();
@@ -634,13 +671,15 @@ int launch_split(const bf16* q, size_t q_stride, const bf16* k, const bf16* vt, 
                  int n_requests, int nh, int nkv, int page_size, float scale, int window, int min_blocks,
                  int n_splits, const float* sink, const AttnExtras* extras, hipStream_t stream) {
   dim3 grid(n_splits, nkv, n_requests), block(4 * MS_WAVE);
-  if (extras)
+  if (extras && extras->value_dim != D)
+    attention_mfma_kernel<D, 1, 4, true, 1, true, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink, *extras);
+  else if (extras)
     attention_mfma_kernel<D, 1, 4, true, 1, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink, *extras);
   else if (sink)
     attention_mfma_kernel<D, 1, 4, true, 1, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink);
   else
     attention_mfma_kernel<D, 1, 4, true, 1, false><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, nullptr);
-  attention_combine_kernel<D><<<dim3(n_requests * nh), dim3(D < 64 ? 64 : D), 0, stream>>>(part_o, part_ml, q_start, ctx, out, out_stride, nh, window, min_blocks, n_splits, extras ? extras->gate : nullptr, extras ? extras->gate_stride : 0, extras ? extras->out_scale : 1.0f);
+  attention_combine_kernel<D><<<dim3(n_requests * nh), dim3(D < 64 ? 64 : D), 0, stream>>>(part_o, part_ml, q_start, ctx, out, out_stride, nh, extras ? extras->value_dim : D, window, min_blocks, n_splits, extras ? extras->gate : nullptr, extras ? extras->gate_stride : 0, extras ? extras->gate_width : 1, extras ? extras->out_scale : 1.0f);
   return ms_launch_status();
 }
 
@@ -656,32 +695,41 @@ extern "C" void ms_attention_mfma_force(int nt, int waves, int dim_shares) {
 }
 
 // Whether the matrix-core kernels take this geometry (else the caller uses the generic kernel).
-extern "C" int ms_attention_mfma_supported(int head_dim, int page_size) {
-  return (head_dim == 32 || head_dim == 64 || head_dim == 128) && page_size > 0 && page_size % 16 == 0;
+// value_dim: the key size, or a smaller multiple of 16.
+extern "C" int ms_attention_mfma_supported(int head_dim, int value_dim, int page_size) {
+  return (head_dim == 32 || head_dim == 64 || head_dim == 128) && page_size > 0 && page_size % 16 == 0 &&
+         value_dim > 0 && value_dim <= head_dim && value_dim % 16 == 0;
+}
+
+// A gate of one number per entry is read four entries at a time.
+static bool gate_fits(const void* gate, long long gate_stride, int gate_width, int value_dim) {
+  if (gate == nullptr || gate_width == 1) return true;
+  return gate_width == value_dim && gate_stride % 4 == 0 && (uintptr_t)gate % 8 == 0;
 }
 
 // General shape.  q [N, >= nh*d] bfloat16 (row stride q_stride), k_pages [P, nkv, page_size, d],
-// vt_pages [P, nkv, d, page_size], block_table int32 [rows, table_stride], table_rows int32 [R] (the table's row
+// vt_pages [P, nkv, value_dim, page_size], block_table int32 [rows, table_stride], table_rows int32 [R] (the table's row
 // of each request; null: request r has row r), q_start int32 [R + 1], context_lens int32 [R] (keys held after
-// this step), out [N, nh*d] (row stride out_stride).  n_tokens = q_start[R] or more, max_q_len the longest
+// this step), out [N, nh*value_dim] (row stride out_stride).  n_tokens = q_start[R] or more, max_q_len the longest
 // portion or more: the launch is sized by these two and n_requests alone, so tokens beyond q_start[R] and
 // requests without tokens cost a block that leaves at once.
 extern "C" int ms_paged_attention_mfma(const void* q, long long q_stride, const void* k_pages, const void* vt_pages,
                                        const int* block_table, int table_stride, const int* table_rows,
                                        const int* q_start, const int* context_lens, void* out, long long out_stride,
                                        int n_requests, int n_tokens, int max_q_len, int num_heads, int num_kv_heads,
-                                       int head_dim, int page_size, float scale, int window, const float* sink,
+                                       int head_dim, int value_dim, int page_size, float scale, int window, const float* sink,
                                        float softcap, const float* slopes, const void* gate, long long gate_stride,
-                                       float out_scale, hipStream_t stream) {
+                                       int gate_width, float out_scale, hipStream_t stream) {
   if (n_requests <= 0 || max_q_len <= 0 || n_tokens <= 0) return MS_OK;
   if (num_heads <= 0 || num_kv_heads <= 0 || num_heads % num_kv_heads || table_stride <= 0) return MS_BAD_ARG;
   if (!(scale > 0.f)) return MS_BAD_ARG;   // maxima are taken of the raw scores
-  if (!ms_attention_mfma_supported(head_dim, page_size)) return MS_UNSUPPORTED;
+  if (!ms_attention_mfma_supported(head_dim, value_dim, page_size)) return MS_UNSUPPORTED;
+  if (!gate_fits(gate, gate_stride, gate_width, value_dim)) return MS_UNSUPPORTED;
   if (q_stride % 8 || out_stride % 4 || ((uintptr_t)q % 16) || ((uintptr_t)out % 8)) return MS_UNSUPPORTED;
   if (n_requests > 65535 || num_kv_heads > 65535) return MS_UNSUPPORTED;
-  const bool changed = softcap > 0.f || slopes != nullptr || gate != nullptr || out_scale != 1.0f;
+  const bool changed = softcap > 0.f || slopes != nullptr || gate != nullptr || out_scale != 1.0f || value_dim != head_dim;
   const AttnExtras ex = {scale, softcap > 0.f ? softcap : 0.f, softcap > 0.f ? 2.0f * 1.4426950408889634f / softcap : 0.f,
-                         slopes, (const bf16*)gate, (size_t)gate_stride, out_scale};
+                         slopes, (const bf16*)gate, (size_t)gate_stride, gate_width, out_scale, value_dim};
   const AttnExtras* extras = changed ? &ex : nullptr;
 #define GO(D, NT, WV, VS) return launch_general<D, NT, WV, VS>((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)vt_pages, block_table, table_stride, table_rows, q_start, context_lens, (bf16*)out, out_stride, n_requests, n_tokens, max_q_len, num_heads, num_kv_heads, page_size, scale, window, sink, extras, stream)
   // Tile width (NT * 16 columns) and waves over a tile's keys.  Few columns (a decode step): one narrow tile
@@ -705,7 +753,7 @@ extern "C" int ms_paged_attention_mfma(const void* q, long long q_stride, const 
   // with a sink the widest tile at head size 64 has no register left for the softmax's other starting point
   if ((sink != nullptr || changed) && head_dim == 64 && nt == 4) nt = 2;
   if (changed && nt == 1) {     // the variants with changed scores: eight waves over a narrow tile's keys, four at 128 dims
-    if (head_dim == 32) vs = 1;
+    if (head_dim == 32 || value_dim != head_dim) vs = 1;
     waves = head_dim == 128 && vs == 1 ? 4 : 8;
   }
   if (g_force_nt) { nt = g_force_nt; waves = g_force_waves; }
@@ -727,28 +775,29 @@ extern "C" int ms_paged_attention_mfma(const void* q, long long q_stride, const 
 
 // Split shape, for long contexts in small batches: every request has exactly one token and the group
 // (num_heads / num_kv_heads) is at most 16; the keys are spread over n_splits blocks and combined.
-// part_o: float [R, nh, n_splits, d], part_ml: float [R, nh, n_splits, 2].  Each request spreads its blocks of
+// part_o: float [R, nh, n_splits, value_dim], part_ml: float [R, nh, n_splits, 2].  Each request spreads its blocks of
 // 32 keys evenly over the n_splits waves, at least min_blocks to a wave, so the launch does not depend on
 // how long the contexts are.
 extern "C" int ms_paged_attention_mfma_decode(const void* q, long long q_stride, const void* k_pages,
                                               const void* vt_pages, const int* block_table, int table_stride,
                                               const int* table_rows, const int* q_start, const int* context_lens, void* out,
                                               long long out_stride, void* part_o, void* part_ml, int n_requests,
-                                              int num_heads, int num_kv_heads, int head_dim, int page_size,
+                                              int num_heads, int num_kv_heads, int head_dim, int value_dim, int page_size,
                                               float scale, int window, int min_blocks, int n_splits, const float* sink,
                                               float softcap, const float* slopes, const void* gate, long long gate_stride,
-                                              float out_scale, hipStream_t stream) {
+                                              int gate_width, float out_scale, hipStream_t stream) {
   if (n_requests <= 0) return MS_OK;
   if (num_heads <= 0 || num_kv_heads <= 0 || num_heads % num_kv_heads || table_stride <= 0) return MS_BAD_ARG;
   if (num_heads / num_kv_heads > 16) return MS_UNSUPPORTED;
   if (!(scale > 0.f)) return MS_BAD_ARG;
-  if (!ms_attention_mfma_supported(head_dim, page_size)) return MS_UNSUPPORTED;
+  if (!ms_attention_mfma_supported(head_dim, value_dim, page_size)) return MS_UNSUPPORTED;
+  if (!gate_fits(gate, gate_stride, gate_width, value_dim)) return MS_UNSUPPORTED;
   if (min_blocks <= 0 || n_splits <= 0 || n_splits > COMBINE_MAX_SPLITS) return MS_BAD_ARG;
   if (q_stride % 8 || out_stride % 4 || ((uintptr_t)q % 16) || ((uintptr_t)out % 8) || ((uintptr_t)part_o % 16)) return MS_UNSUPPORTED;
   if (n_requests > 65535 || num_kv_heads > 65535) return MS_UNSUPPORTED;
-  const bool changed = softcap > 0.f || slopes != nullptr || gate != nullptr || out_scale != 1.0f;
+  const bool changed = softcap > 0.f || slopes != nullptr || gate != nullptr || out_scale != 1.0f || value_dim != head_dim;
   const AttnExtras ex = {scale, softcap > 0.f ? softcap : 0.f, softcap > 0.f ? 2.0f * 1.4426950408889634f / softcap : 0.f,
-                         slopes, (const bf16*)gate, (size_t)gate_stride, out_scale};
+                         slopes, (const bf16*)gate, (size_t)gate_stride, gate_width, out_scale, value_dim};
   const AttnExtras* extras = changed ? &ex : nullptr;
 #define GO(D) return launch_split<D>((const bf16*)q, q_stride, (const bf16*)k_pages, (const bf16*)vt_pages, block_table, table_stride, table_rows, q_start, context_lens, (bf16*)out, out_stride, (float*)part_o, (float*)part_ml, n_requests, num_heads, num_kv_heads, page_size, scale, window, min_blocks, n_splits, sink, extras, stream)
   if (head_dim == 32) GO(32);

@@ -1,6 +1,7 @@
 // Kernels of a feed-forward made of routed experts, all driven by device data so that a step can be captured:
 //   route    per token: softmax over the router's outputs, the `top` largest of (score + correction), their scores;
-//            optionally inside the best groups of neighbouring outputs only, and with the scores divided by their sum
+//            optionally inside the best groups of neighbouring outputs only (a group counts as its best output or as its
+//            two best ones' sum), with the scores divided by their sum, and with a constant factor
 //   align    rows (token, choice) grouped by expert into tiles of TILE rows, each tile of one expert
 //   grouped  out[row] = act(W[expert of the row's tile] . in[row]) for every tile, gathered / scattered by the rows' list;
 //            act: none, the exact gelu, or (matrix cores) the clamped gate over interleaved gate and up features
@@ -40,12 +41,13 @@ __global__ void act_kernel(const T* __restrict__ x, T* __restrict__ out, size_t 
 
 // One wave per token.  Ties go to the lower index.  sigmoid_scores: every score is the sigmoid of its own logit
 // instead of the softmax over all of them.  groups > 0: the outputs form that many equal groups of neighbours, a group
-// counts as its largest (score + correction), and only outputs of the `keep` best groups can be chosen.  normalise: the
-// chosen outputs' scores are divided by (their sum + 1e-20).
+// counts as its largest (score + correction) (group_top 2: as the sum of its two largest), and only outputs of the `keep` best
+// groups can be chosen.  normalise: the chosen outputs' scores are divided by (their sum + 1e-20).  The weights are the
+// scores times weight_scale.
 __global__ void __launch_bounds__(256)
 moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __restrict__ correction, int n_tokens,
                  int n_out, int top, int* __restrict__ ids, float* __restrict__ weights, int sigmoid_scores, int groups,
-                 int keep, int normalise) {
+                 int keep, int group_top, int normalise, float weight_scale) {
   extern __shared__ float s_choice[];     // with groups: [waves][n_out + groups] (score + correction, then the groups' maxima)
   const int lane = threadIdx.x & (MS_WAVE - 1);
   const int n = blockIdx.x * (blockDim.x / MS_WAVE) + threadIdx.x / MS_WAVE;
@@ -90,9 +92,13 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
     for (int g = lane; g < groups; g += MS_WAVE) {
-      float m = -INFINITY;
-      for (int i = 0; i < size; ++i) m = fmaxf(m, choice[g * size + i]);
-      best[g] = m;
+      float m = -INFINITY, second = -INFINITY;
+      for (int i = 0; i < size; ++i) {
+        const float v = choice[g * size + i];
+        second = fmaxf(second, fminf(m, v));
+        m = fmaxf(m, v);
+      }
+      best[g] = group_top == 2 && size > 1 ? m + second : m;
     }
     __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "wavefront");
     __builtin_amdgcn_wave_barrier();
@@ -134,7 +140,7 @@ moe_route_kernel(const float* __restrict__ logits, size_t ld, const float* __res
     for (int i = 0; i < ROUTE_MAX_PER_LANE; ++i)
       if (i * MS_WAVE < n_out && lane + i * MS_WAVE == be) c[i] = -INFINITY;
   }
-  if (lane < top) weights[(size_t)n * top + lane] = normalise ? my_weight / (total + 1e-20f) : my_weight;
+  if (lane < top) weights[(size_t)n * top + lane] = (normalise ? my_weight / (total + 1e-20f) : my_weight) * weight_scale;
 }
 
 // One block.  rows[cap] (cap = tiles * tile): for every tile its rows' flat index n * top + j, or -1; tile_expert[tiles]:
@@ -484,15 +490,17 @@ extern "C" int ms_relu2(const void* x, void* out, long long total, int dtype, hi
 }
 
 extern "C" int ms_moe_route(const float* logits, long long ld, const float* correction, int n_tokens, int n_out, int top,
-                            int* ids, float* weights, int sigmoid_scores, int groups, int keep, int normalise,
-                            hipStream_t stream) {
+                            int* ids, float* weights, int sigmoid_scores, int groups, int keep, int group_top, int normalise,
+                            float weight_scale, hipStream_t stream) {
   if (n_tokens <= 0) return MS_OK;
   if (n_out <= 0 || top <= 0 || top > n_out || groups < 0) return MS_BAD_ARG;
+  if (groups > 0 && group_top != 1 && group_top != 2) return MS_BAD_ARG;
   if (groups > 0 && (n_out % groups || keep <= 0 || keep > groups || top > keep * (n_out / groups))) return MS_BAD_ARG;
   if (n_out > ROUTE_MAX_PER_LANE * MS_WAVE || top > ROUTE_MAX_TOP) return MS_UNSUPPORTED;
   const size_t lds = groups > 0 ? (size_t)4 * (n_out + groups) * sizeof(float) : 0;
   moe_route_kernel<<<(n_tokens + 3) / 4, 256, lds, stream>>>(logits, (size_t)ld, correction, n_tokens, n_out, top, ids,
-                                                             weights, sigmoid_scores, groups, keep, normalise);
+                                                             weights, sigmoid_scores, groups, keep, group_top, normalise,
+                                                             weight_scale);
   return ms_launch_status();
 }
 

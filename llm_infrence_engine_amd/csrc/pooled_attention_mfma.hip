@@ -563,7 +563,7 @@ extern "C" int ms_pooled_attention_mfma(const void* q, long long q_stride, const
       pk_pages == nullptr || pvt_pages == nullptr || pool_table == nullptr)
     return MS_BAD_ARG;
   if (!(scale > 0.f)) return MS_BAD_ARG;
-  if (!ms_attention_mfma_supported(head_dim, page_size)) return MS_UNSUPPORTED;
+  if (!ms_attention_mfma_supported(head_dim, head_dim, page_size)) return MS_UNSUPPORTED;
   if (q_stride % 8 || out_stride % 4 || ((uintptr_t)q % 16) || ((uintptr_t)out % 8)) return MS_UNSUPPORTED;
   if (n_requests > 65535 || num_kv_heads > 65535) return MS_UNSUPPORTED;
   if ((uintptr_t)turn_back % 8) return MS_BAD_ARG;

@@ -7,6 +7,11 @@
 // divided by their root mean square even where no weight is given.  Keys and values may have different sizes.
 // qkv [N, nh * d + nkv * d + nkv * dv]; q and k are rewritten in place.  Norms, logarithm, temperature, angles, sines
 // and cosines are float.
+//
+// ms_qk_span_norm_store: the same place for norms that run over the whole projection: all q heads of a token are divided by
+// one root mean square and multiplied by one weight per entry of the projection, all k heads by another; then the rotation
+// and the store.  Values may be blended on their way into the pages, v <- (1 - lambda) v + lambda first, with another
+// matrix's row of the same token (`first`) and one stored number lambda; the projection's own v stays as it is.
 #include "common.h"
 #include "api.h"
 
@@ -94,6 +99,87 @@ qk_norm_store_kernel(T* __restrict__ qkv, size_t stride, const float* __restrict
   }
 }
 
+// One block per token, V neighbouring entries of a head to a thread and step (V = 8: heads, halves of the rotated part and
+// rows are whole pieces of 16 bytes in bfloat16).  q and k wait in LDS, as floats, between the sums and the rotation.
+template <typename T, int V> struct alignas(sizeof(T) * V < 16 ? sizeof(T) * V : 16) Piece { T v[V]; };
+
+template <typename T, int V>
+__global__ void __launch_bounds__(512)
+qk_span_norm_store_kernel(T* __restrict__ qkv, size_t stride, const float* __restrict__ q_w, const float* __restrict__ k_w,
+                          float eps, const int* __restrict__ positions, const float* __restrict__ inv_freq, int rot_dim,
+                          const T* __restrict__ first, size_t first_stride, const float* __restrict__ lambda,
+                          const int* __restrict__ slots, T* __restrict__ k_pages, T* __restrict__ v_pages, int nh, int nkv,
+                          int d, int dv, int page_size, int v_transposed) {
+  extern __shared__ __align__(16) float s_mem[];     // [rot_dim] cosines, sines; then q and k, [(nh + nkv) * d]
+  __shared__ float red[16];
+  float* cs = s_mem;
+  float* sn = s_mem + rot_dim / 2;
+  float* row_f = s_mem + rot_dim + (4 - rot_dim % 4) % 4;
+  const int n = blockIdx.x, tid = threadIdx.x;
+  T* row = qkv + (size_t)n * stride;
+  const int nq = nh * d, nk = nkv * d, half = rot_dim / 2;
+  typedef Piece<T, V> P;
+  typedef Piece<float, V> F;
+  if (rot_dim > 0) {
+    const float pos = (float)positions[n];
+    for (int i = tid; i < half; i += blockDim.x) sincosf(pos * inv_freq[i], &sn[i], &cs[i]);
+  }
+  float sq = 0.f, sk = 0.f;
+  for (int i = tid * V; i < nq + nk; i += blockDim.x * V) {
+    const P p = *reinterpret_cast<const P*>(row + i);
+    F f;
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < V; ++j) { f.v[j] = to_float(p.v[j]); ss = fmaf(f.v[j], f.v[j], ss); }
+#pragma unroll
+    for (int j = 0; j < V; ++j) row_f[i + j] = f.v[j];
+    if (i < nq) sq += ss; else sk += ss;
+  }
+  sq = block_sum(sq, red);
+  sk = block_sum(sk, red);       // (its barriers also stand between the rows' writes to LDS and their reads)
+  const float iq = 1.0f / sqrtf(sq / (float)nq + eps), ik = 1.0f / sqrtf(sk / (float)nk + eps);
+  const int slot = slots ? slots[n] : -1;
+  const int page = slot >= 0 ? slot / page_size : 0, off = slot >= 0 ? slot % page_size : 0;
+  for (int i = tid * V; i < nq + nk; i += blockDim.x * V) {
+    const bool is_q = i < nq;
+    const int at = is_q ? i : i - nq;       // entry of its projection, head and entry of its head
+    const int head = at / d, e = at - head * d;
+    const float inv = is_q ? iq : ik;
+    const float* w = (is_q ? q_w : k_w) + at;
+    F v;
+#pragma unroll
+    for (int j = 0; j < V; ++j) v.v[j] = row_f[i + j] * inv * w[j];
+    if (e < rot_dim) {                      // (V > 1: a piece lies in one half)
+      const bool low = e < half;
+      const int other = low ? half : -half, pair = low ? e : e - half;
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        const float o = row_f[i + other + j] * inv * w[other + j];
+        const float c = cs[pair + j], s = sn[pair + j];
+        v.v[j] = low ? v.v[j] * c - o * s : v.v[j] * c + o * s;
+      }
+    }
+    P p;
+#pragma unroll
+    for (int j = 0; j < V; ++j) p.v[j] = from_float<T>(v.v[j]);
+    *reinterpret_cast<P*>(row + i) = p;
+    if (!is_q && k_pages && slot >= 0)
+      *reinterpret_cast<P*>(k_pages + (((size_t)page * nkv + head) * page_size + off) * d + e) = p;
+  }
+  if (v_pages && slot >= 0) {
+    const T* vr = row + nq + nk;
+    const T* fr = first ? first + (size_t)n * first_stride : nullptr;
+    const float lam = first ? *lambda : 0.f;
+    for (int i = tid; i < nkv * dv; i += blockDim.x) {
+      T v = vr[i];
+      if (fr) v = from_float<T>(fmaf(lam, to_float(fr[i]), (1.0f - lam) * to_float(v)));
+      const int g = i / dv, e = i - g * dv;
+      if (v_transposed) v_pages[(((size_t)page * nkv + g) * dv + e) * page_size + off] = v;
+      else v_pages[(((size_t)page * nkv + g) * page_size + off) * dv + e] = v;
+    }
+  }
+}
+
 }  // namespace
 
 extern "C" int ms_qk_norm_store(void* qkv, long long stride, const float* q_weight, const float* k_weight, float eps,
@@ -119,6 +205,38 @@ extern "C" int ms_qk_norm_store(void* qkv, long long stride, const float* q_weig
                                                       inv_freq, rot_dim)
   if (dtype == MS_F32) LAUNCH(float);
   else if (dtype == MS_BF16) LAUNCH(bf16);
+  else return MS_BAD_ARG;
+#undef LAUNCH
+  return ms_launch_status();
+}
+
+// q_weight float [nh * d], k_weight float [nkv * d]; first: rows of [nkv * dv] (first_stride apart) and lambda a float on the
+// device, or null.  q and k of one token must fit in LDS as floats.
+extern "C" int ms_qk_span_norm_store(void* qkv, long long stride, const float* q_weight, const float* k_weight, float eps,
+                                     const int* positions, const float* inv_freq, int rot_dim, const void* first,
+                                     long long first_stride, const float* lambda, const int* slots, void* k_pages,
+                                     void* v_pages, int n_tokens, int num_heads, int num_kv_heads, int head_dim,
+                                     int value_dim, int page_size, int v_transposed, int dtype, hipStream_t stream) {
+  if (n_tokens <= 0) return MS_OK;
+  if (num_heads <= 0 || num_kv_heads <= 0 || head_dim <= 0 || value_dim <= 0 || !q_weight || !k_weight) return MS_BAD_ARG;
+  if (rot_dim < 0 || rot_dim % 2 || rot_dim > head_dim || (rot_dim > 0 && (positions == nullptr || inv_freq == nullptr)))
+    return MS_BAD_ARG;
+  if ((first != nullptr) != (lambda != nullptr)) return MS_BAD_ARG;
+  if ((k_pages != nullptr) != (v_pages != nullptr) || (k_pages != nullptr && (slots == nullptr || page_size <= 0)))
+    return MS_BAD_ARG;
+  const size_t lds = ((size_t)(num_heads + num_kv_heads) * head_dim + rot_dim + 4) * sizeof(float);
+  if (lds > 60 * 1024) return MS_UNSUPPORTED;
+  const uintptr_t all = (uintptr_t)qkv | (uintptr_t)k_pages;
+  const bool wide = head_dim % 8 == 0 && (rot_dim / 2) % 8 == 0 && stride % 8 == 0 && all % 16 == 0;
+  dim3 grid(n_tokens), block(n_tokens <= 256 ? 512 : 256);
+#define LAUNCH(T, V)                                                                                                      \
+  qk_span_norm_store_kernel<T, V><<<grid, block, lds, stream>>>((T*)qkv, (size_t)stride, q_weight, k_weight, eps,       \
+                                                                positions, inv_freq, rot_dim, (const T*)first,          \
+                                                                (size_t)first_stride, lambda, slots, (T*)k_pages,       \
+                                                                (T*)v_pages, num_heads, num_kv_heads, head_dim,         \
+                                                                value_dim, page_size, v_transposed)
+  if (dtype == MS_F32) { if (wide) LAUNCH(float, 8); else LAUNCH(float, 1); }
+  else if (dtype == MS_BF16) { if (wide) LAUNCH(bf16, 8); else LAUNCH(bf16, 1); }
   else return MS_BAD_ARG;
 #undef LAUNCH
   return ms_launch_status();

@@ -62,14 +62,15 @@ _SIGNATURES = {
                         _c_int, _c_int, _c_ptr],
     "ms_paged_attention_generic": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
                                    _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ll, _c_float, _c_int, _c_int,
-                                   _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ll, _c_float, _c_int, _c_ptr],
-    "ms_attention_mfma_supported": [_c_int, _c_int],
+                                   _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ll, _c_int, _c_float, _c_int, _c_ptr],
+    "ms_attention_mfma_supported": [_c_int, _c_int, _c_int],
     "ms_paged_attention_mfma": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll,
-                                _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr,
-                                _c_float, _c_ptr, _c_ptr, _c_ll, _c_float, _c_ptr],
+                                _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float, _c_int, _c_ptr,
+                                _c_float, _c_ptr, _c_ptr, _c_ll, _c_int, _c_float, _c_ptr],
     "ms_paged_attention_mfma_decode": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
-                                       _c_ll, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
-                                       _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ll, _c_float, _c_ptr],
+                                       _c_ll, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_float,
+                                       _c_int, _c_int, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_ll, _c_int, _c_float,
+                                       _c_ptr],
     "ms_argmax": [_c_ptr, _c_ll, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr],
     "ms_sample": [_c_ptr, _c_ll, _c_int, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int,
                   _c_ptr],
@@ -104,11 +105,13 @@ _SIGNATURES = {
     "ms_latent_attention": [_c_ptr, _c_ll, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr,
                             _c_ptr, _c_ll, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ll, _c_float, _c_int, _c_int,
                             _c_ptr],
-    "ms_rms_norm_add": [_c_ptr, _c_ll, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_int, _c_int, _c_int,
-                        _c_ptr],
+    "ms_rms_norm_add": [_c_ptr, _c_ll, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_float, _c_ptr,
+                        _c_int, _c_int, _c_int, _c_ptr],
     "ms_add_rows": [_c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_ptr],
     "ms_qk_norm_store": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_float, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int,
                          _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr, _c_int, _c_int, _c_ptr],
+    "ms_qk_span_norm_store": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_float, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ll, _c_ptr, _c_ptr,
+                              _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "ms_selective_scan": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_ptr, _c_ptr,
                           _c_ptr, _c_ptr, _c_ll, _c_int, _c_int, _c_int, _c_int, _c_ptr],
     "ms_gelu": [_c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr],
@@ -116,7 +119,8 @@ _SIGNATURES = {
     "ms_streams_max": [],
     "ms_streams": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_float,
                    _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int, _c_ptr],
-    "ms_moe_route": [_c_ptr, _c_ll, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_ptr],
+    "ms_moe_route": [_c_ptr, _c_ll, _c_ptr, _c_int, _c_int, _c_int, _c_ptr, _c_ptr, _c_int, _c_int, _c_int, _c_int, _c_int,
+                     _c_float, _c_ptr],
     "ms_layer_norm": [_c_ptr, _c_ptr, _c_int, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_ptr, _c_int, _c_int, _c_float, _c_int, _c_int, _c_ptr],
     "ms_side_gate": [_c_ptr, _c_ll, _c_ptr, _c_ptr, _c_ll, _c_int, _c_ptr, _c_int, _c_int, _c_int, _c_ptr],
     "ms_mingru_chunk": [],
@@ -772,6 +776,16 @@ def qkv_rope_store(x: torch.Tensor, norm_weight: torch.Tensor, eps: float, w_qkv
     return q
 
 
+def _gate_of(gate: Optional[torch.Tensor], q: torch.Tensor, num_heads: int, dv: int):
+    """(row stride, numbers per head) of an attention's output gate: one number per head, or one per entry of the result."""
+    if gate is None:
+        return 0, 1
+    stride = _rows2d(gate, "gate", q.dtype)
+    if gate.shape != (q.shape[0], num_heads) and gate.shape != (q.shape[0], num_heads * dv):
+        raise ValueError(f"gate must be [{q.shape[0]}, {num_heads}] or [{q.shape[0]}, {num_heads * dv}], got {list(gate.shape)}")
+    return stride, gate.shape[1] // num_heads
+
+
 def paged_attention_generic(q: torch.Tensor, k_pages: torch.Tensor, v_pages: torch.Tensor, block_table: torch.Tensor,
                             token_req: torch.Tensor, positions: torch.Tensor, out: torch.Tensor, num_heads: int,
                             scale: float, window: Optional[int] = None, v_transposed: bool = False,
@@ -790,7 +804,8 @@ def paged_attention_generic(q: torch.Tensor, k_pages: torch.Tensor, v_pages: tor
     keys (the value pages say which; out is then [N, nh * that size]).  ``sink`` float [nh]: exp(sink[h]) joins the
     denominator of head h's softmax.  ``softcap`` > 0: a scaled score s becomes softcap * tanh(s / softcap).  ``slopes``
     float [nh]: slopes[h] * (positions[n] - key's position) is taken off the score (after the cap).  ``gate`` [N, nh] (rows
-    may be slices): head h's result is multiplied by sigmoid(gate[n, h]); ``out_scale`` multiplies every result."""
+    may be slices): head h's result is multiplied by sigmoid(gate[n, h]), or [N, nh * value size]: every entry of the results
+    by a sigmoid of its own; ``out_scale`` multiplies every result."""
     _check(k_pages, "k_pages")
     P, nkv, page_size, d = k_pages.shape
     _check(v_pages, "v_pages", k_pages.dtype, (P, nkv, None, None))
@@ -816,20 +831,19 @@ def paged_attention_generic(q: torch.Tensor, k_pages: torch.Tensor, v_pages: tor
         raise ValueError(f"{num_heads} query heads cannot share {nkv} key/value heads")
     if slopes is not None:
         _check(slopes, "slopes", torch.float32, (num_heads,))
-    gate_stride = _rows2d(gate, "gate", q.dtype, num_heads) if gate is not None else 0
-    if gate is not None and gate.shape[0] != N:
-        raise ValueError("gate must have a row per token")
+    gate_stride, gate_width = _gate_of(gate, q, num_heads, dv)
     _call("ms_paged_attention_generic", q.data_ptr(), q.stride(0) if N > 1 else q.shape[1], k_pages.data_ptr(),
           v_pages.data_ptr(), block_table.data_ptr(), block_table.shape[1], _ptr(table_rows), _ptr(n_live_tokens),
           token_req.data_ptr(), positions.data_ptr(),
           out.data_ptr(), num_heads * dv, N, num_heads, nkv, d, dv, page_size, P, float(scale), int(window or 0),
-          int(v_transposed), _ptr(sink), float(softcap or 0.0), _ptr(slopes), _ptr(gate), gate_stride, float(out_scale),
-          _code(q.dtype), _stream())
+          int(v_transposed), _ptr(sink), float(softcap or 0.0), _ptr(slopes), _ptr(gate), gate_stride, gate_width,
+          float(out_scale), _code(q.dtype), _stream())
     return out
 
 
-def attention_mfma_supported(head_dim: int, page_size: int) -> bool:
-    return bool(_get("ms_attention_mfma_supported")(head_dim, page_size))
+def attention_mfma_supported(head_dim: int, page_size: int, value_dim: Optional[int] = None) -> bool:
+    """Whether the matrix-core attention takes these sizes (``value_dim`` None: the key size)."""
+    return bool(_get("ms_attention_mfma_supported")(head_dim, head_dim if value_dim is None else value_dim, page_size))
 
 
 SPLIT_BLOCKS = 512         # blocks a split decode step's attention aims to put on the chip (two to a CU)
@@ -851,7 +865,8 @@ def paged_attention_mfma(q: torch.Tensor, k_pages: torch.Tensor, vt_pages: torch
                          table_rows: Optional[torch.Tensor] = None, sink: Optional[torch.Tensor] = None,
                          softcap: float = 0.0, slopes: Optional[torch.Tensor] = None,
                          gate: Optional[torch.Tensor] = None, out_scale: float = 1.0) -> torch.Tensor:
-    """Matrix-core attention, bfloat16.  k_pages [P, nkv, page_size, d], vt_pages [P, nkv, d, page_size];
+    """Matrix-core attention, bfloat16.  k_pages [P, nkv, page_size, d], vt_pages [P, nkv, value size, page_size]
+    (the key size or a smaller multiple of 16);
     request r owns tokens q_start[r]..q_start[r+1]-1, holds context_lens[r] keys after this step and has row
     ``table_rows[r]`` of ``block_table`` (row r without ``table_rows``).  ``max_q_len`` and ``max_context_len``
     are upper bounds; tokens from q_start[R] on belong to no request, a request may have no token.  A small
@@ -863,17 +878,16 @@ def paged_attention_mfma(q: torch.Tensor, k_pages: torch.Tensor, vt_pages: torch
         _check(sink, "sink", torch.float32, (num_heads,))
     if slopes is not None:
         _check(slopes, "slopes", torch.float32, (num_heads,))
-    gate_stride = _rows2d(gate, "gate", torch.bfloat16, num_heads) if gate is not None else 0
-    if gate is not None and gate.shape[0] != q.shape[0]:
-        raise ValueError("gate must have a row per token")
-    more = (float(softcap or 0.0), _ptr(slopes), _ptr(gate), gate_stride, float(out_scale))
     P, nkv, page_size, d = k_pages.shape
-    _check(vt_pages, "vt_pages", torch.bfloat16, (P, nkv, d, page_size))
+    _check(vt_pages, "vt_pages", torch.bfloat16, (P, nkv, None, page_size))
+    dv = vt_pages.shape[2]
+    gate_stride, gate_width = _gate_of(gate, q, num_heads, dv)
+    more = (float(softcap or 0.0), _ptr(slopes), _ptr(gate), gate_stride, gate_width, float(out_scale))
     _check(q, "q", torch.bfloat16, contiguous=False)
     N = q.shape[0]
     if q.dim() != 2 or q.stride(1) != 1 or q.shape[1] < num_heads * d:
         raise ValueError(f"q must be [N, >= {num_heads * d}] with unit stride along rows, got {list(q.shape)}")
-    _check(out, "out", torch.bfloat16, (N, num_heads * d))
+    _check(out, "out", torch.bfloat16, (N, num_heads * dv))
     _check(block_table, "block_table", torch.int32)
     R = context_lens.numel()
     _check(q_start, "q_start", torch.int32, (R + 1,))
@@ -898,16 +912,16 @@ def paged_attention_mfma(q: torch.Tensor, k_pages: torch.Tensor, vt_pages: torch
         # allow (one request of 100,000 keys, two kv heads: 61 us in 16 splits, 24.4 in 64, 23.4 in 128, 27 in 256).
         most = MAX_SPLITS * (1 if max_context_len <= 16384 else (2 if max_context_len <= 65536 else 8))
         n_splits = max(1, min(most, SPLIT_BLOCKS // max(1, R * nkv)))
-        part_o = torch.empty((R, num_heads, n_splits, d), dtype=torch.float32, device=q.device)
+        part_o = torch.empty((R, num_heads, n_splits, dv), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((R, num_heads, n_splits, 2), dtype=torch.float32, device=q.device)
         _call("ms_paged_attention_mfma_decode", q.data_ptr(), q_stride, k_pages.data_ptr(), vt_pages.data_ptr(),
               block_table.data_ptr(), block_table.shape[1], _ptr(table_rows), q_start.data_ptr(), context_lens.data_ptr(),
-              out.data_ptr(), num_heads * d, part_o.data_ptr(), part_ml.data_ptr(), R, num_heads, nkv, d, page_size, float(scale),
+              out.data_ptr(), num_heads * dv, part_o.data_ptr(), part_ml.data_ptr(), R, num_heads, nkv, d, dv, page_size, float(scale),
               int(window or 0), MIN_BLOCKS_PER_SPLIT, n_splits, _ptr(sink), *more, _stream())
     else:
         _call("ms_paged_attention_mfma", q.data_ptr(), q_stride, k_pages.data_ptr(), vt_pages.data_ptr(),
               block_table.data_ptr(), block_table.shape[1], _ptr(table_rows), q_start.data_ptr(), context_lens.data_ptr(),
-              out.data_ptr(), num_heads * d, R, N, max_q_len, num_heads, nkv, d, page_size, float(scale), int(window or 0),
+              out.data_ptr(), num_heads * dv, R, N, max_q_len, num_heads, nkv, d, dv, page_size, float(scale), int(window or 0),
               _ptr(sink), *more, _stream())
     return out
 
@@ -951,20 +965,19 @@ def paged_attention(q: torch.Tensor, kv, ctx, out: torch.Tensor, num_heads: int,
                     out_scale: float = 1.0) -> torch.Tensor:
     """Attention of a step's tokens (``ctx``: its StepContext) over a run's pages (``kv``: its KVView).
     bfloat16 with transposed value pages and a head size the matrix-core kernel has goes there; everything
-    else (float32, other head sizes, values of another size than keys, small pages) goes to the generic kernel.
+    else (float32, other key or value sizes, small pages) goes to the generic kernel.
     ``sink`` float [num_heads]: exp(sink[h]) joins the denominator of head h's softmax."""
     d, page_size = kv.k_pages.shape[3], kv.k_pages.shape[2]
     dv = kv.v_pages.shape[2] if kv.v_transposed else kv.v_pages.shape[3]
-    if dv != d:
-        return paged_attention_generic(q, kv.k_pages, kv.v_pages, kv.block_table, ctx.token_req, ctx.positions, out,
-                                       num_heads, scale, window, kv.v_transposed, kv.table_rows, ctx.n_live_tokens, sink,
-                                       softcap, slopes, gate, out_scale)
-    if q.dtype == torch.bfloat16 and not (kv.v_transposed and attention_mfma_supported(d, page_size)):
-        _say_once(("attention", d, page_size),
-                  f"bfloat16 attention with head size {d} and pages of {page_size} tokens runs on the vector-ALU kernel: "
-                  f"the matrix-core kernel takes head sizes 32, 64 and 128 with pages of a multiple of 16")
-    if (q.dtype == torch.bfloat16 and kv.v_transposed and attention_mfma_supported(d, page_size)
-            and q.data_ptr() % 16 == 0 and (q.shape[0] == 1 or q.stride(0) % 8 == 0)):
+    takes = kv.v_transposed and attention_mfma_supported(d, page_size, dv)
+    if q.dtype == torch.bfloat16 and not takes:
+        _say_once(("attention", d, dv, page_size),
+                  f"bfloat16 attention with keys of {d}, values of {dv} and pages of {page_size} tokens runs on the vector-ALU "
+                  f"kernel: the matrix-core kernel takes keys of 32, 64 and 128, values of that size or a smaller multiple of "
+                  f"16, and pages of a multiple of 16")
+    by_entry = gate is not None and gate.shape[1] != num_heads
+    if (q.dtype == torch.bfloat16 and takes and q.data_ptr() % 16 == 0 and (q.shape[0] == 1 or q.stride(0) % 8 == 0)
+            and not (by_entry and (gate.data_ptr() % 8 or (q.shape[0] > 1 and gate.stride(0) % 4)))):
         return paged_attention_mfma(q, kv.k_pages, kv.v_pages, kv.block_table, ctx.q_start, ctx.context_lens, out,
                                     num_heads, scale, ctx.max_q_len, ctx.max_context_len, window, kv.table_rows, sink,
                                     softcap, slopes, gate, out_scale)
@@ -1379,25 +1392,45 @@ def latent_attention(q: torch.Tensor, kv, ctx, out: torch.Tensor, scale: float, 
 
 
 # ------------------------------------------------------------------------------------------------ norms after a sublayer
-def rms_norm_add(y: torch.Tensor, w_post: torch.Tensor, eps_post: float, x: torch.Tensor,
+def rms_norm_add(y, w_post: torch.Tensor, eps_post: float, x: torch.Tensor,
                  w_next: Optional[torch.Tensor] = None, eps_next: float = 0.0,
                  out: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """x += w_post * y / sqrt(mean(y^2) + eps_post), in place on the float residual stream x [N, H]; y [N, H] (rows may be
-    slices of wider rows) is a sublayer's output.  With ``out`` [N, H] also out = w_next * x / sqrt(mean(x^2) + eps_next),
-    the norm the next sublayer reads, from the same pass."""
+    slices of wider rows) is a sublayer's output, or (base [N, H] or None, part float [N * k, H], weights float [N, k]) for
+    base[n] + sum_j weights[n, j] part[n k + j].  With ``out`` [N, H] also what the next sublayer reads, from the same pass:
+    out = w_next * x / sqrt(mean(x^2) + eps_next), or without ``w_next`` out = x, rounded."""
     _check(x, "x", torch.float32)
     N, H = x.shape
-    ys = _rows2d(y, "y", None, H)
-    if y.shape[0] != N:
+    part = weights = None
+    top = 0
+    if isinstance(y, tuple):
+        y, part, weights = y
+        _check(weights, "weights", torch.float32, (N, None))
+        top = weights.shape[1]
+        _check(part, "part", torch.float32, (N * top, H))
+    ys = _rows2d(y, "y", None, H) if y is not None else 0
+    if y is not None and y.shape[0] != N:
         raise ValueError(f"y has {y.shape[0]} rows, x {N}")
     _check(w_post, "w_post", torch.float32, (H,))
     ocode = 0
     if out is not None:
         _check(out, "out", None, (N, H))
-        _check(w_next, "w_next", torch.float32, (H,))
+        if w_next is not None:
+            _check(w_next, "w_next", torch.float32, (H,))
         ocode = _code(out.dtype)
-    _call("ms_rms_norm_add", y.data_ptr(), ys, _code(y.dtype), w_post.data_ptr(), float(eps_post), x.data_ptr(),
-          _ptr(w_next) if out is not None else None, float(eps_next), _ptr(out), ocode, N, H, _stream())
+    _call("ms_rms_norm_add", _ptr(y), ys, _code(y.dtype) if y is not None else F32, _ptr(part), _ptr(weights), top,
+          w_post.data_ptr(), float(eps_post), x.data_ptr(), _ptr(w_next) if out is not None else None, float(eps_next),
+          _ptr(out), ocode, N, H, _stream())
+    return out
+
+
+def round_rows(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """out [N, H] = the float stream x, rounded to out's type."""
+    _check(x, "x", torch.float32)
+    N, H = x.shape
+    _check(out, "out", None, (N, H))
+    _call("ms_rms_norm_add", None, 0, F32, None, None, 0, None, 0.0, x.data_ptr(), None, 0.0, out.data_ptr(), _code(out.dtype),
+          N, H, _stream())
     return out
 
 
@@ -1451,6 +1484,47 @@ def qk_norm_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim
           int(every), _ptr(slot_mapping), _ptr(k_pages), _ptr(v_pages), N, num_heads, num_kv_heads, head_dim, value_dim,
           page_size, int(bool(v_transposed)), int(bool(unit_norm)), _ptr(inv_freq) if rot_dim else None, int(rot_dim),
           _code(qkv.dtype), _stream())
+    return qkv
+
+
+def qk_span_norm_store(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, value_dim: int,
+                       q_weight: torch.Tensor, k_weight: torch.Tensor, eps: float, positions: Optional[torch.Tensor] = None,
+                       inv_freq: Optional[torch.Tensor] = None, rot_dim: int = 0, first: Optional[torch.Tensor] = None,
+                       blend: Optional[torch.Tensor] = None, slot_mapping: Optional[torch.Tensor] = None,
+                       k_pages: Optional[torch.Tensor] = None, v_pages: Optional[torch.Tensor] = None,
+                       v_transposed: bool = False) -> torch.Tensor:
+    """In place on ``qkv`` [N, nh d + nkv d + nkv dv]: all q heads of a token are divided by one root mean square and
+    multiplied by q_weight float [nh d], all k heads by another and k_weight [nkv d]; then the rotation of ``qk_norm_store``;
+    then k and v go into the pages, v as (1 - blend) v + blend first where ``first`` [N, nkv dv] (rows may be slices; v's type)
+    and ``blend`` (one float on the device) are given.  The v part of ``qkv`` stays as it is."""
+    width = (num_heads + num_kv_heads) * head_dim + num_kv_heads * value_dim
+    stride = _rows2d(qkv, "qkv", None, width)
+    N = qkv.shape[0]
+    _check(q_weight, "q_weight", torch.float32, (num_heads * head_dim,))
+    _check(k_weight, "k_weight", torch.float32, (num_kv_heads * head_dim,))
+    if rot_dim:
+        if rot_dim % 2 or not 0 < rot_dim <= head_dim:
+            raise ValueError(f"{rot_dim} rotated entries must be even and within the head's {head_dim}")
+        _check(positions, "positions", torch.int32, (N,))
+        _check(inv_freq, "inv_freq", torch.float32, (rot_dim // 2,))
+    first_stride = 0
+    if first is not None:
+        first_stride = _rows2d(first, "first", qkv.dtype, num_kv_heads * value_dim)
+        if first.shape[0] != N:
+            raise ValueError(f"first has {first.shape[0]} rows, qkv {N}")
+        _check(blend, "blend", torch.float32)
+        if blend.numel() != 1:
+            raise ValueError("blend is one number")
+    page_size = 0
+    if k_pages is not None:
+        _check(k_pages, "k_pages", qkv.dtype, (None, num_kv_heads, None, head_dim))
+        page_size = k_pages.shape[2]
+        _check(v_pages, "v_pages", qkv.dtype, _v_shape(k_pages, v_transposed, value_dim))
+        _check(slot_mapping, "slot_mapping", torch.int32, (N,))
+    _call("ms_qk_span_norm_store", qkv.data_ptr(), stride, q_weight.data_ptr(), k_weight.data_ptr(), float(eps), _ptr(positions),
+          _ptr(inv_freq) if rot_dim else None, int(rot_dim), _ptr(first), first_stride, _ptr(blend) if first is not None else None,
+          _ptr(slot_mapping), _ptr(k_pages), _ptr(v_pages), N, num_heads, num_kv_heads, head_dim, value_dim, page_size,
+          int(bool(v_transposed)), _code(qkv.dtype), _stream())
     return qkv
 
 
@@ -1510,12 +1584,13 @@ def relu2(x: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
 
 
 def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int, n_out: Optional[int] = None,
-              scores: str = "softmax", groups=None, normalise: bool = False):
+              scores: str = "softmax", groups=None, normalise: bool = False, group_top: int = 1, weight_scale: float = 1.0):
     """Scores = softmax(logits[:, :n_out]) (``scores`` "sigmoid": every logit's own sigmoid); the ``top`` largest of
     scores + correction are chosen (the lower index on a tie).  Returns (ids int32 [N, top], their scores float [N, top]).
     logits float [N, >= n_out].  ``groups`` (count, keep): the outputs form ``count`` equal groups of neighbours, a group
-    counts as its largest score + correction, and only outputs of the ``keep`` best groups can be chosen.  ``normalise``:
-    the chosen scores are divided by (their sum + 1e-20)."""
+    counts as its largest score + correction (``group_top`` 2: as the sum of its two largest), and only outputs of the ``keep``
+    best groups can be chosen.  ``normalise``: the chosen scores are divided by (their sum + 1e-20); ``weight_scale`` multiplies
+    what is returned."""
     if scores not in ("softmax", "sigmoid"):
         raise ValueError(f"router scores are 'softmax' or 'sigmoid', not {scores!r}")
     ld = _rows2d(logits, "logits", torch.float32)
@@ -1528,10 +1603,12 @@ def moe_route(logits: torch.Tensor, correction: Optional[torch.Tensor], top: int
     count, keep = groups if groups is not None else (0, 0)
     if groups is not None and (count <= 0 or n_out % count or not 0 < keep <= count or top > keep * (n_out // count)):
         raise ValueError(f"top {top} of {n_out} outputs within {keep} of {count} equal groups")
+    if group_top not in (1, 2):
+        raise ValueError(f"a group counts as its best output or as its two best ones' sum, not as its {group_top} best")
     ids = torch.empty((N, top), dtype=torch.int32, device=logits.device)
     weights = torch.empty((N, top), dtype=torch.float32, device=logits.device)
     _call("ms_moe_route", logits.data_ptr(), ld, _ptr(correction), N, n_out, top, ids.data_ptr(), weights.data_ptr(),
-          int(scores == "sigmoid"), count, keep, int(normalise), _stream())
+          int(scores == "sigmoid"), count, keep, int(group_top), int(normalise), float(weight_scale), _stream())
     return ids, weights
 
 

@@ -9,8 +9,11 @@ the softmax's denominator; it has no key and no value and is not scaled; ``sink=
 every head and no tensor (one is added to the denominator).  ``softcap`` c: a scaled score s becomes c tanh(s / c).
 ``slope_base`` b: head h of H takes slope_h (i - j) off the score of key j for query i, slope_h = 2^(-b (h + 1) / H) (after the
 cap).  ``gate``: a projection [heads, hidden] (tensor "gate") whose sigmoid multiplies every head's result, one number per
-token and head, before the output projection; it rides on the packed q/k/v product.  ``out_scale`` multiplies the heads'
-results.  ``names``: the tensors' names after the prefix, {"q", "k", "v", "o", "sink", "gate"} -> name; biases are the weight's
+token and head, before the output projection (``gate="entry"``: [heads * value size, hidden], one number per entry of the
+concatenated heads); it rides on the packed q/k/v product.  ``value_blend``: layers of a model blend their values with those of
+the first such layer.  "first": this is that layer, whose values of the step's tokens the others find in ``ctx.shared``;
+"blend": v <- (1 - lambda) v + lambda first, with a stored number lambda (tensor "blend"), on the way into the pages.
+``out_scale`` multiplies the heads' results.  ``names``: the tensors' names after the prefix, {"q", "k", "v", "o", "sink", "gate", "blend"} -> name; biases are the weight's
 name with ".bias" for ".weight", or the weight's name followed by ``bias_suffix``.
 """
 from __future__ import annotations
@@ -24,7 +27,8 @@ from ..weights.spec import TensorSpec
 from .base import CacheNeed, KVNeed, Mixer, PageTensor, register_part
 
 _NAMES = {"q": "q_proj.weight", "k": "k_proj.weight", "v": "v_proj.weight", "o": "o_proj.weight", "sink": "sink",
-          "gate": "gate"}
+          "gate": "gate", "blend": "blend"}
+FIRST_VALUES = ("gqa_attention", "first_values")     # the key of ``StepContext.shared`` they lie under
 
 
 class GQAttention(Mixer):
@@ -33,8 +37,8 @@ class GQAttention(Mixer):
     def __init__(self, prefix: str, position, hidden_size: int, num_heads: int, num_kv_heads: int, head_dim: int,
                  scale: float, qkv_bias: bool = True, out_bias: bool = False, window: Optional[int] = None,
                  value_dim: Optional[int] = None, sink=False, names=None, softcap: Optional[float] = None,
-                 slope_base: Optional[float] = None, gate: bool = False, out_scale: float = 1.0,
-                 bias_suffix: Optional[str] = None):
+                 slope_base: Optional[float] = None, gate=False, out_scale: float = 1.0,
+                 bias_suffix: Optional[str] = None, value_blend: Optional[str] = None):
         if num_heads % num_kv_heads:
             raise ValueError(f"{num_heads} query heads cannot share {num_kv_heads} key/value heads")
         if not 0 < head_dim <= 256:
@@ -58,7 +62,15 @@ class GQAttention(Mixer):
             raise ValueError("softcap must be positive")
         self.softcap = float(softcap) if softcap is not None else 0.0
         self.slope_base = float(slope_base) if slope_base is not None else None
+        if gate not in (False, True, "entry"):
+            raise ValueError(f"gate is False, True (one number per head) or 'entry', got {gate!r}")
         self.gate, self.out_scale, self.bias_suffix = bool(gate), float(out_scale), bias_suffix
+        self.gate_width = num_heads * (self.value_dim if gate == "entry" else 1)
+        if value_blend not in (None, "first", "blend"):
+            raise ValueError(f"value_blend is None, 'first' or 'blend', got {value_blend!r}")
+        if value_blend == "blend" and not getattr(position, "takes_value_blend", False):
+            raise ValueError("blended values need a position encoding that stores them (one with takes_value_blend)")
+        self.value_blend = value_blend
         self.names = dict(_NAMES, **dict(names or {}))
         self.slopes = self.w_gate_rows = None
 
@@ -82,7 +94,9 @@ class GQAttention(Mixer):
         if self.sink:
             specs.append(TensorSpec(p + self.names["sink"], (self.num_heads,), "bias"))
         if self.gate:
-            specs.append(TensorSpec(p + self.names["gate"], (self.num_heads, H)))
+            specs.append(TensorSpec(p + self.names["gate"], (self.gate_width, H)))
+        if self.value_blend == "blend":
+            specs.append(TensorSpec(p + self.names["blend"], (), "bias"))
         if self.position is not None:
             specs += self.position.tensor_specs()
         return specs
@@ -92,8 +106,9 @@ class GQAttention(Mixer):
         by_name = {s.name: s for s in GQAttention.tensor_specs(self)}
         p = self.prefix
         w = [get(by_name[p + self.names[n]]) for n in ("q", "k", "v")]
-        if self.gate:       # the gate's rows ride on the packed product, after q, k and v; rows of zeros make the
-            w.append(get(by_name[p + self.names["gate"]]))      # product's rows a multiple of 16 bytes, as the matrix-core attention reads q
+        if self.gate:       # the gate's rows ride on the packed product, after q, k and v
+            w.append(get(by_name[p + self.names["gate"]]))
+            # rows of zeros make the product's rows a multiple of 16 bytes, as the matrix-core attention reads q
             pad = (-sum(t.shape[0] for t in w)) % 8
             if pad:
                 w.append(torch.zeros(pad, self.hidden_size, dtype=w[0].dtype, device=w[0].device))
@@ -109,6 +124,7 @@ class GQAttention(Mixer):
         self.sink_w = get(by_name[p + self.names["sink"]]) if self.sink else None
         if self.zero_sink:
             self.sink_w = torch.zeros(self.num_heads, dtype=torch.float32, device=rt.device)
+        self.blend_w = get(by_name[p + self.names["blend"]]) if self.value_blend == "blend" else None
         if self.slope_base is not None:
             H = self.num_heads
             self.slopes = torch.tensor([2.0 ** (-self.slope_base * (h + 1) / H) for h in range(H)], dtype=torch.float64) \
@@ -123,8 +139,10 @@ class GQAttention(Mixer):
         if self.value_dim == self.head_dim:
             return KVNeed(self.num_kv_heads, self.head_dim, self.window, transpose_values_at=16,
                           transpose_values_in=torch.bfloat16)
+        narrow = self.value_dim < self.head_dim and self.value_dim % 16 == 0      # what those kernels take beside equal sizes
         return CacheNeed((PageTensor("k", self.num_kv_heads, self.head_dim),
-                          PageTensor("v", self.num_kv_heads, self.value_dim)), self.window)
+                          PageTensor("v", self.num_kv_heads, self.value_dim, 16 if narrow else None,
+                                     torch.bfloat16 if narrow else None)), self.window)
 
     # ---- step
     def forward(self, h, ctx, kv, state):
@@ -134,8 +152,8 @@ class GQAttention(Mixer):
         if kv is None:
             raise RuntimeError("attention needs a key/value cache view")
         nh, nkv, d, dv = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
-        if self.gate:
-            return self._forward_gated(h, ctx, kv, x)
+        if self.gate or self.value_blend:
+            return self._forward_packed(h, ctx, kv, x)
         q = None
         if self.position is not None and dv == d:
             q = self.position.project_encode_store(h, self.w_qkv, self.b_qkv, nh, nkv, d, ctx, kv)
@@ -158,24 +176,34 @@ class GQAttention(Mixer):
                             self.out_scale)
         return linear.linear_residual(out, self.w_o, self.b_o, x)
 
-    def _forward_gated(self, h, ctx, kv, x):
-        """With an output gate: one product for q, k, v and the gate's numbers; the position encoding works on the first
-        columns, the attention kernel reads the last ones."""
+    def _blending(self, qkv, ctx):
+        """{} or the keyword that has the position encoding blend the values with the first such layer's."""
+        if self.value_blend is None:
+            return {}
+        if self.value_blend == "first":       # the projection's own v, which nothing overwrites while the step runs
+            ctx.shared[FIRST_VALUES] = qkv[:, qkv.shape[1] - self.num_kv_heads * self.value_dim:]
+            return {}
+        return {"blend": (ctx.shared[FIRST_VALUES], self.blend_w)}
+
+    def _forward_packed(self, h, ctx, kv, x):
+        """With an output gate or blended values: one product for q, k, v and the gate's numbers; the position encoding works
+        on the first columns, the attention kernel reads the last ones."""
         nh, nkv, d, dv = self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim
         width = (nh + nkv) * d + nkv * dv
         proj = linear.linear(h, self.w_qkv, bias=self.b_qkv)
         qkv = proj[:, :width]
+        blending = self._blending(qkv, ctx)
         if self.position is None:
             if kv.store:
                 ops.qk_norm_store(qkv, nh, nkv, d, dv, None, None, 0.0, slot_mapping=kv.slot_mapping, k_pages=kv.k_pages,
                                   v_pages=kv.v_pages, v_transposed=kv.v_transposed)
         elif dv != d or getattr(self.position, "takes_value_dim", False):
-            self.position.encode_and_store(qkv, nh, nkv, d, ctx, kv, value_dim=dv)
+            self.position.encode_and_store(qkv, nh, nkv, d, ctx, kv, value_dim=dv, **blending)
         else:
-            self.position.encode_and_store(qkv, nh, nkv, d, ctx, kv)
+            self.position.encode_and_store(qkv, nh, nkv, d, ctx, kv, **blending)
         out = self.rt.empty(ctx.num_tokens, nh * dv)
         ops.paged_attention(qkv, kv, ctx, out, nh, self.scale, self.window, self.sink_w, self.softcap, self.slopes,
-                            proj[:, width:width + nh], self.out_scale)
+                            proj[:, width:width + self.gate_width] if self.gate else None, self.out_scale)
         return linear.linear_residual(out, self.w_o, self.b_o, x)
 
 

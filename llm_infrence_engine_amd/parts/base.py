@@ -209,6 +209,7 @@ class Norm(Part):
     # "rms" (x over its root mean square) or "layer" (mean taken off first): the norm is that, times ``weight``, plus
     # ``bias`` (None: none), with ``eps``, and a kernel that has the row at hand may take it itself.  None: only ``forward``.
     statistic: Optional[str] = None
+    settles_writes = False      # as ``Block.settles_writes``, of ``forward``'s delta
 
     def lazy(self, x: torch.Tensor, delta: Optional[torch.Tensor] = None, rows: Optional[torch.Tensor] = None,
              write_back: bool = True):
@@ -304,6 +305,9 @@ class Block(Part):
 
     takes: Dict[str, str] = {}
     optional: Tuple[str, ...] = ()
+    # True: ``pending`` may be an object with ``add_into(x)``, a write that is more than an addend (a normed sum, a write into
+    # several streams), and the block carries it out with whatever pass it makes; else the model does so first
+    settles_writes = False
 
     def __init__(self, **built):
         unknown = set(built) - set(self.takes)

@@ -6,8 +6,11 @@ it as an epilogue) or hands the addend on, and the sum is fused into the norm th
 own last addend on as ``pending``."""
 from __future__ import annotations
 
+from dataclasses import dataclass
+from typing import Any
+
 from ..kernels import ops
-from .base import Block, register_part
+from .base import Block, Norm, register_part
 
 
 class PreNormResidual(Block):
@@ -74,6 +77,43 @@ class SandwichResidual(Block):
         return None
 
 
+@dataclass
+class NormedAddend:
+    """x <- x + norm(y), still to be carried out: ``y`` a sublayer's output (as ``RMSNorm.add_normed`` takes it)."""
+
+    y: Any
+    norm: Norm
+
+    def add_into(self, x):
+        self.norm.add_normed(x, self.y)
+
+
+class PostNormResidual(Block):
+    """x <- x + post1(mixer(x));  x <- x + post2(feed_forward(x)): sublayers read the residual stream as it is and only what
+    they return is normalised.  The sum into x and x in the activations' type for the next sublayer are one pass, over layers
+    too: a layer hands its last sum on as ``pending``.  Without a feed-forward the layer is its first line."""
+
+    takes = {"position": "position", "mixer": "mixer", "mixer_post_norm": "norm", "feed_forward": "feed_forward",
+             "feed_forward_post_norm": "norm"}
+    optional = ("position", "feed_forward", "feed_forward_post_norm")
+    settles_writes = True
+
+    def forward(self, x, pending, ctx, kv, state):
+        if isinstance(pending, NormedAddend):
+            h = pending.norm.add_normed(x, pending.y, plain=True)
+        else:
+            if hasattr(pending, "add_into"):
+                pending.add_into(x)
+            elif pending is not None:
+                ops.residual_add(x, pending)
+            h = x if self.rt.dtype == x.dtype else ops.round_rows(x, self.rt.empty(*x.shape))
+        y = self.mixer.forward(h, ctx, kv, state)
+        if self.feed_forward is None:
+            return NormedAddend(y, self.mixer_post_norm)
+        h = self.mixer_post_norm.add_normed(x, y, plain=True)
+        return NormedAddend(self.feed_forward.forward_deferred(h, ctx), self.feed_forward_post_norm)
+
+
 class ScaledPreNormResidual(Block):
     """x <- x + s1 o mixer(norm1(x));  x <- x + s2 o feed_forward(norm2(x));  then, if the layer has one, the token's own
     input (``token_input``) into x.  s1, s2 (``mixer_scale``, ``feed_forward_scale``; optional) are stored vectors.  Every
@@ -108,4 +148,5 @@ class ScaledPreNormResidual(Block):
 register_part("block", "pre_norm_residual", PreNormResidual)
 register_part("block", "pre_norm_scaled_residual", ScaledPreNormResidual)
 register_part("block", "sandwich_residual", SandwichResidual)
+register_part("block", "post_norm_residual", PostNormResidual)
 register_part("block", "parallel_residual", ParallelResidual)

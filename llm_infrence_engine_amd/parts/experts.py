@@ -10,8 +10,9 @@ s to their results, in float, before the activation).  The first ``experts`` out
 that every token runs, weighted by sigmoid(W_sg h), one number per token, or (``shared_gate`` False) as it is.
 ``activation`` "clamped_glu" with ``limit`` and ``alpha``: g = min(gate(h), limit), u = clamp(up(h), -limit, limit), an expert
 is down(g sigmoid(alpha g) (u + 1)); the shared expert is of the same form with ``shared_limit``.  ``groups`` (count, keep):
-the outputs form ``count`` equal groups of neighbours, a group counts as its largest s + correction, and only outputs of the
-``keep`` best groups can be chosen.  ``normalise``: the chosen weights are divided by their sum (+ 1e-20).
+the outputs form ``count`` equal groups of neighbours, a group counts as its largest s + correction (``group_top`` 2: as the sum
+of its two largest), and only outputs of the ``keep`` best groups can be chosen.  ``normalise``: the chosen weights are divided by
+their sum (+ 1e-20); ``weight_scale`` multiplies them.
 
 Nothing here waits for the device: the tokens' choices are grouped by expert into tiles on the device, and the experts'
 products run tile by tile over a launch whose size depends on the sizes alone, so a step can be captured."""
@@ -31,7 +32,8 @@ class RoutedExperts(FeedForward):
     def __init__(self, prefix: str, hidden_size: int, expert_ff: int, experts: int, top: int, identity: int = 0,
                  shared_ff: int = 0, activation: str = "gelu", scores: str = "softmax", correction: bool = True,
                  weight_on: str = "output", groups=None, normalise: bool = False, limit: Optional[float] = None,
-                 alpha: float = 1.702, shared_limit: Optional[float] = None, shared_gate: bool = True):
+                 alpha: float = 1.702, shared_limit: Optional[float] = None, shared_gate: bool = True, group_top: int = 1,
+                 weight_scale: float = 1.0):
         if activation not in ("gelu", "swiglu", "clamped_glu"):
             raise ValueError(f"no activation {activation!r} for routed experts; there are 'gelu', 'swiglu' and 'clamped_glu'")
         if activation == "clamped_glu" and (limit is None or (shared_ff and shared_limit is None)):
@@ -50,6 +52,9 @@ class RoutedExperts(FeedForward):
         self.experts, self.identity, self.top, self.shared_ff = experts, identity, top, shared_ff
         self.activation, self.scores, self.has_correction, self.weight_on = activation, scores, bool(correction), weight_on
         self.groups, self.normalise = (tuple(groups) if groups is not None else None), bool(normalise)
+        self.group_top, self.weight_scale = int(group_top), float(weight_scale)
+        if self.group_top not in (1, 2):
+            raise ValueError(f"a group counts as its best output or as its two best ones' sum, not as its {group_top} best")
         if self.groups is not None:
             count, keep = self.groups
             n_out = experts + identity
@@ -100,7 +105,8 @@ class RoutedExperts(FeedForward):
         """(ids [N, top], weights float [N, top] or None, the chosen experts' rows float [N * top, W], router's logits)."""
         N, W, E = h.shape[0], self.hidden_size, self.experts
         logits = linear.linear(h, self.w_router, out_dtype=torch.float32)
-        ids, weights = ops.moe_route(logits, self.correction, self.top, E + self.identity, self.scores, self.groups, self.normalise)
+        ids, weights = ops.moe_route(logits, self.correction, self.top, E + self.identity, self.scores, self.groups, self.normalise,
+                                     self.group_top, self.weight_scale)
         rows, tile_expert = ops.moe_align(ids, E, ops.moe_tile_choice(ids.numel(), E, (W, self.expert_ff), h.dtype))
         mid = None
         if self.activation == "clamped_glu" and h.dtype == torch.bfloat16 and W % 32 == 0:

@@ -92,7 +92,8 @@ class Model:
 
     def forward_hidden(self, ctx: StepContext, caches: List[RunCache]):
         """Embedding and all runs of the order: the float residual stream ([N, H], or [N, S, H] where the model has S
-        copies of it) and what the last run has still to write into it (an addend, a ``StreamsWrite``, or None)."""
+        copies of it) and what the last run has still to write into it (an addend, a write that the final norm carries out
+        itself, or None)."""
         x = self.embedding.forward(ctx)
         kept = x.clone() if self.pass_entry is not None and self.pass_entry.keeps_embedding else None
         pending = None
@@ -106,8 +107,18 @@ class Model:
                 new = self.pass_entry.forward(x, kept, run.opens_pass)
                 x = x if new is None else new
             c = caches[i]
+            pending = self._settled(x, pending, self.layers[run.layer])
             pending = self.layers[run.layer].forward(x, pending, ctx, c.kv, c.state)
-        return x, pending
+        return x, self._settled(x, pending, self.final_norm)
+
+    @staticmethod
+    def _settled(x, pending, reader):
+        """``pending`` as ``reader`` (a block or the final norm) takes it: a write that is more than an addend is carried out
+        now if the reader does not do that itself."""
+        if hasattr(pending, "add_into") and not reader.settles_writes:
+            pending.add_into(x)
+            return None
+        return pending
 
     def head_logits(self, x: torch.Tensor, pending: Optional[torch.Tensor], rows: torch.Tensor) -> torch.Tensor:
         """Final norm and head on the rows ``rows`` (int32) of what ``forward_hidden`` returned; x is left as it is."""

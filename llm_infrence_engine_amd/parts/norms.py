@@ -1,7 +1,8 @@
 """RMS norm: y = gain * (offset + weight) * x * rsqrt(mean(x^2) + eps), computed in float on the float residual stream.
 ``offset`` is 0 for a scale stored as it is and 1 for one stored around zero; ``gain`` is a constant of the layer (the
-weight of a normed sublayer in the residual sum, say); both are folded into the weight once, in float, when the weights
-are loaded.  ``add_normed`` is the norm of a sublayer's *output* on its way into the residual stream.
+weight of a normed sublayer in the residual sum, or the logits' scale); both are folded into the weight once, in float, when the weights
+are loaded.  ``add_normed`` is the norm of a sublayer's *output* on its way into the residual stream, and with it what the next
+sublayer reads.
 
 The reference computes the reduction in float, casts back and multiplies by the weight in the model's
 type (src/miniserve/model.py:69-73); here the weight is applied in float too and the result is rounded once.
@@ -41,10 +42,16 @@ class RMSNorm(Norm):
         return ops.rms_norm(x, self.weight, self.eps, out, delta=delta, rows=rows, write_back=write_back)
 
 
-    def add_normed(self, x, y, then: "RMSNorm" = None):
+    def add_normed(self, x, y, then: "RMSNorm" = None, plain: bool = False):
         """x += this norm of y, in place on the float residual stream (y: a sublayer's output, any activation type or
-        float).  With ``then`` (another norm of the same width) also returns that norm of the new x, from the same
+        float, or a sum left to do, as ``FeedForward.forward_deferred`` returns it).  With ``then`` (another norm of the same
+        width) also returns that norm of the new x, with ``plain`` the new x itself in the activations' type, from the same
         pass over the rows."""
+        if plain:
+            if self.rt.dtype == x.dtype:
+                ops.rms_norm_add(y, self.weight, self.eps, x)
+                return x
+            return ops.rms_norm_add(y, self.weight, self.eps, x, out=self.rt.empty(x.shape[0], self.size))
         if then is None:
             ops.rms_norm_add(y, self.weight, self.eps, x)
             return None

@@ -149,13 +149,16 @@ def yarn_frequencies(dims: int, base: float, scaling=None):
 
 
 def scaled_frequencies(dims: int, base: float, scaling=None) -> torch.Tensor:
-    """f_i = base^(-2 i / dims) for i < dims / 2, in double.  ``scaling`` {"factor", "low", "high", "original"} stretches
+    """f_i = base^(-2 i / dims) for i < dims / 2, in double.  ``scaling`` {"factor"} divides all of them by the factor;
+    ``scaling`` {"factor", "low", "high", "original"} stretches
     the long waves: with a wavelength l = 2 pi / f below original / high, f stays; above original / low, f / factor; in
     between, with s = (original / l - low) / (high - low), the blend (1 - s) f / factor + s f."""
     i = torch.arange(0, dims // 2, dtype=torch.float64)
     f = float(base) ** (-2.0 * i / max(1, dims))
     if scaling is None:
         return f
+    if set(scaling) == {"factor"}:
+        return f / float(scaling["factor"])
     factor, low, high, original = (float(scaling[k]) for k in ("factor", "low", "high", "original"))
     if high == low:
         raise ValueError("frequency scaling needs high != low")
@@ -170,18 +173,26 @@ class QKNormRotaryHalf(PositionEncoding):
     the root) and, with ``weighted``, multiplied by a weight of its kind (``q_norm_name`` / ``k_norm_name`` [head_dim], shared
     by the heads); then, with ``dims`` > 0, entry i and entry i + dims / 2 of the head's first ``dims`` entries turn by
     position * f_i (``scaled_frequencies``); the rest pass.  Keys and values may differ in size.  Norm, angles, sines and
-    cosines are float; one kernel also stores k and v into the pages."""
+    cosines are float; one kernel also stores k and v into the pages.
+
+    ``over`` "projection" (``heads``: the numbers of query and of key heads): all query heads of a token are divided by one
+    root mean square and multiplied by one weight per entry of the projection, all key heads by another.  Values may then be
+    blended on their way into the pages: ``blend`` = (first, lambda) of ``encode_and_store``, v <- (1 - lambda) v + lambda first."""
 
     takes_value_dim = True
 
     def __init__(self, prefix: str, head_dim: int, eps: float, weighted: bool = True, dims: int = 0, base: float = 10000.0,
-                 scaling=None, q_norm_name: str = "q.norm", k_norm_name: str = "k.norm"):
+                 scaling=None, q_norm_name: str = "q.norm", k_norm_name: str = "k.norm", over: str = "head", heads=None):
+        if over not in ("head", "projection") or (over == "projection" and (heads is None or not weighted)):
+            raise ValueError("a norm runs over a 'head' or, with weights and the numbers of heads given, the 'projection'")
         if dims % 2 or not 0 <= dims <= head_dim:
             raise ValueError(f"{dims} rotated entries must be even and within the head's {head_dim}")
         self.prefix, self.head_dim, self.eps, self.weighted = prefix, head_dim, float(eps), bool(weighted)
         self.dims, self.base = int(dims), float(base)
         self.scaling = dict(scaling) if scaling is not None else None
         self.q_norm_name, self.k_norm_name = q_norm_name, k_norm_name
+        self.takes_value_blend = over == "projection"
+        self.spans = tuple(n * head_dim for n in heads) if over == "projection" else (head_dim, head_dim)
         self.q_weight = self.k_weight = self.inv_freq = None
 
     def tensor_specs(self):
@@ -189,8 +200,8 @@ class QKNormRotaryHalf(PositionEncoding):
             return []
         from ..weights.spec import TensorSpec
 
-        return [TensorSpec(self.prefix + self.q_norm_name, (self.head_dim,), "norm"),
-                TensorSpec(self.prefix + self.k_norm_name, (self.head_dim,), "norm")]
+        return [TensorSpec(self.prefix + self.q_norm_name, (self.spans[0],), "norm"),
+                TensorSpec(self.prefix + self.k_norm_name, (self.spans[1],), "norm")]
 
     def load(self, get, rt):
         self.rt = rt
@@ -199,8 +210,15 @@ class QKNormRotaryHalf(PositionEncoding):
         if self.dims:
             self.inv_freq = scaled_frequencies(self.dims, self.base, self.scaling).to(torch.float32).to(rt.device)
 
-    def encode_and_store(self, qkv, num_heads, num_kv_heads, head_dim, ctx, kv, value_dim=None):
+    def encode_and_store(self, qkv, num_heads, num_kv_heads, head_dim, ctx, kv, value_dim=None, blend=None):
         store = kv is not None and kv.store
+        if self.takes_value_blend:
+            first, weight = blend if blend is not None else (None, None)
+            ops.qk_span_norm_store(qkv, num_heads, num_kv_heads, head_dim, head_dim if value_dim is None else value_dim,
+                                   self.q_weight, self.k_weight, self.eps, ctx.positions, self.inv_freq, self.dims, first, weight,
+                                   kv.slot_mapping if store else None, kv.k_pages if store else None,
+                                   kv.v_pages if store else None, bool(store and kv.v_transposed))
+            return
         ops.qk_norm_store(qkv, num_heads, num_kv_heads, head_dim, head_dim if value_dim is None else value_dim,
                           self.q_weight, self.k_weight, self.eps, ctx.positions, 0.0, 1,
                           kv.slot_mapping if store else None, kv.k_pages if store else None,

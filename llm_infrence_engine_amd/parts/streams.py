@@ -68,6 +68,7 @@ class HyperConnectedPreNorm(Block):
     takes = {"position": "position", "mixer_norm": "norm", "mixer": "mixer", "mixer_link": "stream_link",
              "feed_forward_norm": "norm", "feed_forward": "feed_forward", "feed_forward_link": "stream_link"}
     optional = ("position", "feed_forward_norm", "feed_forward", "feed_forward_link")
+    settles_writes = True
 
     def __init__(self, **built):
         super().__init__(**built)
@@ -89,6 +90,8 @@ class HyperConnectedPreNorm(Block):
 
 class SummedStreams(Norm):
     """A norm (``norm``: its ``PartSpec``, or a built one's) of the sum of the streams, for a model's end."""
+
+    settles_writes = True
 
     def __init__(self, prefix: str, streams: int, norm):
         self.streams = streams
