@@ -30,7 +30,9 @@ Gidurax and Qwen2, ``--design silizen`` for the Silizen decoder (attention besid
 beside the delta rule, a token-shifted recurrence; one norm per layer, feed-forwards gated with the tanh gelu) beside
 Gemadra and Qwen2, ``--design gositar`` for the Gositar decoder (latent attention over all keys, a residual stream of four
 copies, squared-relu feed-forwards and routed clamped ones in turn) beside Gemadra, whose attention it shares, Kuvazen,
-whose experts are the closest, and Qwen2.
+whose experts are the closest, and Qwen2, ``--design kisusun`` for the Kisusun decoder (capped and gated attention with a sink,
+windowed in three layers of four, norms on the sublayers' outputs, gated feed-forwards and routed clamped ones in turn) beside
+Silizen, whose attention is the closest, Gositar, whose experts it shares, and Qwen2.
 """
 from __future__ import annotations
 
@@ -277,7 +279,8 @@ def run_design(eng, a):
     from llm_infrence_engine_amd.config import config_from_dict, preset
 
     beside = {"gemadra": ["qwen2"], "gidurax": ["gemadra", "qwen2"], "kuvazen": ["gidurax", "qwen2"],
-              "silizen": ["gemadra", "qwen2"], "gositar": ["gemadra", "kuvazen", "qwen2"]}[a.design]
+              "silizen": ["gemadra", "qwen2"], "gositar": ["gemadra", "kuvazen", "qwen2"],
+              "kisusun": ["silizen", "gositar", "qwen2"]}[a.design]
     out = {"design": a.design, "beside": ",".join(beside), "layers": a.design_layers, "dtype": "bf16", "data": "synthetic",
            "prefill_tokens": PREFILL_TOKENS, "prompt_len": a.prompt_len, "sizes": {}}
     for size in a.design_sizes.split(","):
@@ -317,15 +320,16 @@ def run_design(eng, a):
 
 def main() -> int:
     ap = argparse.ArgumentParser(description=__doc__.split("\n\n")[0])
-    ap.add_argument("--design", choices=["gemadra", "gidurax", "kuvazen", "silizen", "gositar"], default=None,
+    ap.add_argument("--design", choices=["gemadra", "gidurax", "kuvazen", "silizen", "gositar", "kisusun"], default=None,
                     help="measure this design beside the closest existing ones (Gemadra beside Qwen2; Gidurax beside "
-                         "Gemadra and Qwen2; Kuvazen beside Gidurax and Qwen2; Silizen beside Gemadra and Qwen2; Gositar beside Gemadra, Kuvazen and Qwen2) at equal sizes instead of the default workload")
+                         "Gemadra and Qwen2; Kuvazen beside Gidurax and Qwen2; Silizen beside Gemadra and Qwen2; Gositar beside Gemadra, Kuvazen and Qwen2; "
+                         "Kisusun beside Silizen, Gositar and Qwen2) at equal sizes instead of the default workload")
     ap.add_argument("--design-layers", type=int, default=4, help="layers of each model in a --design run")
     ap.add_argument("--design-sizes", default="0.5b,7b", help="widths of a --design run (0.5b, 7b)")
     ap.add_argument("--design-part", choices=["all", "prefill", "decode"], default="all",
                     help="a --design run's prompt step or its decode steps alone (for profiles)")
-    ap.add_argument("--design-only", choices=["gemadra", "gidurax", "kuvazen", "silizen", "gositar", "qwen2"], default=None,
-                    help="one of the two models of a --design run alone (for profiles)")
+    ap.add_argument("--design-only", choices=["gemadra", "gidurax", "kuvazen", "silizen", "gositar", "kisusun", "qwen2"], default=None,
+                    help="one of the models of a --design run alone (for profiles)")
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=256)
     ap.add_argument("--warmup", type=int, default=16)

@@ -122,10 +122,16 @@ __device__ __forceinline__ void load_values(ValueBlock<CT>& b, const bf16* __res
 // but only D / VS of the output's dims, so it reads all keys and 1 / VS of the values.  A compute unit draws
 // its data at a small fraction of the chip's rate, so when a step has fewer tiles than the chip has units this
 // shortens the longest chain without a second kernel; the blocks write disjoint dims and share nothing.
-// EXTRA: the scores are changed on their way into the softmax: a scaled score x becomes cap * tanh(x / cap) (cap > 0),
+// EXTRA = CHANGED: the scores are changed on their way into the softmax: a scaled score x becomes cap * tanh(x / cap) (cap > 0),
 // then slope * (the key's distance from the query) is taken off it, one slope per query head; at the end every head's
 // result is multiplied by out_scale and by the sigmoid of a gate, one number per token and head or one per entry.  Such scores are kept
 // in log2 units from the start, and the block's maxima are those of the changed scores.
+// EXTRA = BOUNDED: as CHANGED with a cap of at most BOUNDED_CAP and no slopes.  Such scores lie in [-cap, cap], whose
+// exponentials and their sums and products with values are well inside float's range, so the softmax needs no running
+// maximum: the reference stays where it starts (0; for the wave that holds a positive sink, the sink).
+constexpr int PLAIN = 0, CHANGED = 1, BOUNDED = 2;
+constexpr float BOUNDED_CAP = 60.f;
+
 struct AttnExtras {
   float scale;               // of the raw scores, natural units
   float cap;                 // 0: no cap
@@ -148,8 +154,8 @@ constexpr bool extra_variant() {
 
 // NARROW: values have fewer dims than keys (a multiple of 16); the tiles of 16 dims past them are neither read nor
 // multiplied, which a branch that is the same for the whole launch decides.
-template <int D, int NT, int WAVES, bool SPLIT, int VS, bool SINK, bool EXTRA = false, bool NARROW = false>
-__global__ void __launch_bounds__(WAVES * MS_WAVE, (NT > 1 && !EXTRA ? 2 : 1))
+template <int D, int NT, int WAVES, bool SPLIT, int VS, bool SINK, int EXTRA = PLAIN, bool NARROW = false>
+__global__ void __launch_bounds__(WAVES * MS_WAVE, (NT > 1 && EXTRA != CHANGED && !(NARROW && D == 128) ? 2 : 1))
 attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* __restrict__ k_pages,
                       const bf16* __restrict__ vt_pages, const int* __restrict__ block_table, int table_stride,
                       const int* __restrict__ table_rows, const int* __restrict__ q_start,
@@ -264,11 +270,12 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
 
   // this lane's columns
   int pos[NT];   // -1: an idle column (sees no key; its result is not written)
-  float slope[EXTRA ? NT : 1];
+  float slope[EXTRA == CHANGED ? NT : 1];
   const float sl2 = EXTRA ? 1.0f : scale_log2e;   // what turns a kept score into log2 units
   // the fields the loop reads, as scalars of their own (the struct itself stays in the kernel's arguments)
   const float ex_scale = ex.scale, ex_cap = ex.cap, ex_arg = ex.exp_arg;
   const float* const ex_slopes = ex.slopes;
+  const float raw_arg = ex.scale * ex.exp_arg, cap2 = ex.cap * 1.4426950408889634f;     // BOUNDED: log2 units
   bf16x8 qv[NT][D / 32];
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
@@ -276,7 +283,7 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
     const int cc = min(c, ncols - 1);
     const int tok = q0 + cc / rep, head = g * rep + cc % rep;
     pos[t] = c < ncols ? start_pos + cc / rep : -1;
-    if (EXTRA) slope[t] = ex_slopes ? ex_slopes[head] : 0.f;
+    if (EXTRA == CHANGED) slope[t] = ex_slopes ? ex_slopes[head] : 0.f;
     const bf16* qp = q + (size_t)tok * q_stride + (size_t)head * D + kq * 8;
 #pragma unroll
     for (int s = 0; s < D / 32; ++s) qv[t][s] = *reinterpret_cast<const bf16x8*>(qp + s * 32);
@@ -296,7 +303,7 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
   for (int i = 0; i < 8; ++i) ones[i] = (__bf16)1.0f;
 #pragma unroll
   for (int t = 0; t < NT; ++t) {
-    m[t] = -INFINITY;
+    m[t] = EXTRA == BOUNDED ? 0.f : -INFINITY;
     lvec[t] = 0.f;
     if (SUMS_BY_MATRIX) lsum[t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -310,8 +317,10 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
     for (int t = 0; t < NT; ++t) {
       const int cc = min(c0 + t * 16 + col16, ncols - 1);
       m[t] = sink[g * rep + cc % rep] * 1.4426950408889634f;
-      lvec[t] = kq == 0 ? 1.0f : 0.f;
-      if (SUMS_BY_MATRIX) lsum[t] = f32x4{1.f, 1.f, 1.f, 1.f};
+      float one = 1.0f;
+      if (EXTRA == BOUNDED) { one = fast_exp2(fminf(m[t], 0.f)); m[t] = fmaxf(m[t], 0.f); }
+      lvec[t] = kq == 0 ? one : 0.f;
+      if (SUMS_BY_MATRIX) lsum[t] = f32x4{one, one, one, one};
     }
   }
 
@@ -369,7 +378,7 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
         s[u][t] = acc;
       }
 
-    if (EXTRA) {
+    if (EXTRA == CHANGED) {
       // slope * (pos - key) = slope * (pos - base - 4 kq) - slope * (16 u + i): one product per column, then constants
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
@@ -400,72 +409,91 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
 
     const bool unmasked = full_tile && base + 31 <= first_pos && (window <= 0 || base > key_hi - window);
     bf16x8 p[NT];
-    float corr[NT], bmax[NT];
-    bool moved = false;
-    // the block's maxima of the raw scores (the scale is positive, so they are the maxima of the scaled ones
-    // too); one branch for the whole tile, so that what follows is straight-line code for all its columns
-    if (unmasked) {
-#pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        float bm = -INFINITY;
-#pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) bm = fmaxf(bm, s[u][t][i]);
-        bmax[t] = bm;
-      }
-    } else {
-#pragma unroll
-      for (int t = 0; t < NT; ++t) {
-        float bm = -INFINITY;
-#pragma unroll
-        for (int u = 0; u < 2; ++u)
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const int key = base + u * 16 + kq * 4 + i;
-            const bool see = key <= pos[t] && (window <= 0 || key > pos[t] - window);
-            const float v = see ? s[u][t][i] : -INFINITY;
-            s[u][t][i] = v;
-            bm = fmaxf(bm, v);
-          }
-        bmax[t] = bm;
-      }
-    }
     float m_safe[NT];
+    if constexpr (EXTRA != BOUNDED) {
+      float corr[NT], bmax[NT];
+      bool moved = false;
+      // the block's maxima of the raw scores (the scale is positive, so they are the maxima of the scaled ones
+      // too); one branch for the whole tile, so that what follows is straight-line code for all its columns
+      if (unmasked) {
 #pragma unroll
-    for (int t = 0; t < NT; ++t) {
-      float bm = bmax[t];
-      bm = fmaxf(bm, __shfl_xor(bm, 16, MS_WAVE));
-      bm = fmaxf(bm, __shfl_xor(bm, 32, MS_WAVE));
-      bm *= sl2;
-      // m is the reference that the exponents are taken against, not necessarily the maximum: it follows the
-      // maximum only when that has run ahead by more than REF_SLACK (a factor 2^REF_SLACK in the terms, far
-      // inside float's range), so that the accumulators are rescaled rarely.  Any reference gives the same
-      // softmax; all lanes of a column decide alike because bm is the same in all of them.
-      const bool step = bm > m[t] + REF_SLACK;
-      const float m_new = step ? bm : m[t];
-      corr[t] = step ? fast_exp2(m[t] - m_new) : 1.0f;   // m = -inf: 0
-      moved |= step;
-      m[t] = m_new;
-      m_safe[t] = m_new == -INFINITY ? 0.f : m_new;
-    }
-    if (NT == 1 || __builtin_amdgcn_ballot_w64(moved) != 0) {   // the same branch for the whole wave
+        for (int t = 0; t < NT; ++t) {
+          float bm = -INFINITY;
+#pragma unroll
+          for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) bm = fmaxf(bm, s[u][t][i]);
+          bmax[t] = bm;
+        }
+      } else {
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+          float bm = -INFINITY;
+#pragma unroll
+          for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const int key = base + u * 16 + kq * 4 + i;
+              const bool see = key <= pos[t] && (window <= 0 || key > pos[t] - window);
+              const float v = see ? s[u][t][i] : -INFINITY;
+              s[u][t][i] = v;
+              bm = fmaxf(bm, v);
+            }
+          bmax[t] = bm;
+        }
+      }
 #pragma unroll
       for (int t = 0; t < NT; ++t) {
-        if (SUMS_BY_MATRIX) lsum[t] *= corr[t]; else lvec[t] *= corr[t];
+        float bm = bmax[t];
+        bm = fmaxf(bm, __shfl_xor(bm, 16, MS_WAVE));
+        bm = fmaxf(bm, __shfl_xor(bm, 32, MS_WAVE));
+        bm *= sl2;
+        // m is the reference that the exponents are taken against, not necessarily the maximum: it follows the
+        // maximum only when that has run ahead by more than REF_SLACK (a factor 2^REF_SLACK in the terms, far
+        // inside float's range), so that the accumulators are rescaled rarely.  Any reference gives the same
+        // softmax; all lanes of a column decide alike because bm is the same in all of them.
+        const bool step = bm > m[t] + REF_SLACK;
+        const float m_new = step ? bm : m[t];
+        corr[t] = step ? fast_exp2(m[t] - m_new) : 1.0f;   // m = -inf: 0
+        moved |= step;
+        m[t] = m_new;
+        m_safe[t] = m_new == -INFINITY ? 0.f : m_new;
+      }
+      if (NT == 1 || __builtin_amdgcn_ballot_w64(moved) != 0) {   // the same branch for the whole wave
 #pragma unroll
-        for (int c = 0; c < CT; ++c) o[c][t] *= corr[t];
+        for (int t = 0; t < NT; ++t) {
+          if (SUMS_BY_MATRIX) lsum[t] *= corr[t]; else lvec[t] *= corr[t];
+#pragma unroll
+          for (int c = 0; c < CT; ++c) o[c][t] *= corr[t];
+        }
       }
     }
     // column by column, so that the products of one column run on the matrix cores while the next column's
     // exponentials are taken
 #pragma unroll
     for (int t = 0; t < NT; ++t) {
+      if (EXTRA == BOUNDED) {     // cap tanh(x / cap) = cap - 2 cap / (2^(x arg) + 1)
+        const float top = cap2 - m[t];
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            s[u][t][i] = fmaf(-2.0f * cap2, __builtin_amdgcn_rcpf(fast_exp2(s[u][t][i] * raw_arg) + 1.0f), top);
+        if (!unmasked) {
+#pragma unroll
+          for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              const int key = base + u * 16 + kq * 4 + i;
+              if (key > pos[t] || (window > 0 && key <= pos[t] - window)) s[u][t][i] = -INFINITY;
+            }
+        }
+      }
 #pragma unroll
       for (int u = 0; u < 2; ++u)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float e = fast_exp2(fmaf(s[u][t][i], sl2, -m_safe[t]));
+          const float e = EXTRA == BOUNDED ? fast_exp2(s[u][t][i]) : fast_exp2(fmaf(s[u][t][i], sl2, -m_safe[t]));
           if (!SUMS_BY_MATRIX) lvec[t] += e;
           p[t][u * 4 + i] = (__bf16)e;
         }
@@ -494,6 +522,66 @@ attention_mfma_kernel(const bf16* __restrict__ q, size_t q_stride, const bf16* _
       l[t] = lvec[t] + __shfl_xor(lvec[t], 16, MS_WAVE);
       l[t] += __shfl_xor(l[t], 32, MS_WAVE);
     }
+  }
+  // The variants that change their scores share the end out: each wave merges, gates and writes a part of the dims.
+  constexpr bool SHARED_END = EXTRA != PLAIN && WAVES > 1 && CT % WAVES == 0;
+  if constexpr (SHARED_END) {
+    constexpr int OWN = CT / WAVES;
+    const bool by_entry = !SPLIT && ex.gate && ex.gate_width != 1;
+    bf16x4 gv[NT][OWN];
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      if (kq == 0) { sm_m[wave][t][col16] = m[t]; sm_l[wave][t][col16] = l[t]; }
+#pragma unroll
+      for (int c = 0; c < CT; ++c)
+        if (c / OWN != wave) sm_o[wave < c / OWN ? wave : wave - 1][c][t][lane] = o[c][t];
+      if (by_entry && pos[t] >= 0) {      // the gate's numbers are on their way while the waves wait for each other
+        const int c = c0 + t * 16 + col16;
+        const bf16* gp = ex.gate + (size_t)(q0 + c / rep) * ex.gate_stride + (size_t)(g * rep + c % rep) * DV + dim0 + kq * 4;
+#pragma unroll
+        for (int j = 0; j < OWN; ++j)
+          if (!NARROW || wave * OWN + j < live) gv[t][j] = *reinterpret_cast<const bf16x4*>(gp + (wave * OWN + j) * 16);
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < NT; ++t) {
+      float big = -INFINITY, den = 0.f, f[WAVES];
+#pragma unroll
+      for (int w = 0; w < WAVES; ++w) { f[w] = sm_m[w][t][col16]; big = fmaxf(big, f[w]); }
+      const float safe = big == -INFINITY ? 0.f : big;
+#pragma unroll
+      for (int w = 0; w < WAVES; ++w) { f[w] = fast_exp2(f[w] - safe); den = fmaf(f[w], sm_l[w][t][col16], den); }
+      if (pos[t] < 0) continue;
+      const int col = c0 + t * 16 + col16;
+      const int tok = q0 + col / rep, head = g * rep + col % rep;
+      const size_t slot = SPLIT ? ((size_t)r * nh + head) * n_splits + bx : 0;
+      float inv = 1.0f;
+      if (SPLIT) {
+        if (kq == 0 && wave == 0) { part_ml[slot * 2] = big; part_ml[slot * 2 + 1] = den; }
+      } else {
+        inv = ex.out_scale / den;
+        if (ex.gate && !by_entry) inv *= fast_sigmoid(__bfloat162float(ex.gate[(size_t)tok * ex.gate_stride + head]));
+      }
+#pragma unroll
+      for (int c = 0; c < CT; ++c) {
+        if (c / OWN != wave || (NARROW && c >= live)) continue;
+        f32x4 sum = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int w = 0; w < WAVES; ++w)
+          sum += (w == c / OWN ? o[c][t] : sm_o[w < c / OWN ? w : w - 1][c][t][lane]) * f[w];
+        if (SPLIT) {
+          *reinterpret_cast<f32x4*>(part_o + slot * DV + kq * 4 + c * 16) = sum;
+        } else {
+          bf16x4 w4;
+#pragma unroll
+          for (int i = 0; i < 4; ++i)
+            w4[i] = (__bf16)(by_entry ? sum[i] * inv * fast_sigmoid((float)gv[t][c % OWN][i]) : sum[i] * inv);
+          *reinterpret_cast<bf16x4*>(out + (size_t)tok * out_stride + (size_t)head * DV + dim0 + kq * 4 + c * 16) = w4;
+        }
+      }
+    }
+    return;
   }
   if (WAVES > 1) {
     // merge the waves' partial results (each relative to its own maximum) in wave order
@@ -626,6 +714,8 @@ inline int page_shift_of(int page_size) {   // log2 of a power of two, else -1
   return sh;
 }
 
+inline bool bounded_scores(const AttnExtras& ex) { return ex.cap > 0.f && ex.cap <= BOUNDED_CAP && ex.slopes == nullptr; }
+
 template <int D, int NT, int WAVES, int VS>
 int launch_general(const bf16* q, size_t q_stride, const bf16* k, const bf16* vt, const int* table, int table_stride,
                    const int* table_rows, const int* q_start, const int* ctx, bf16* out, size_t out_stride,
@@ -643,19 +733,22 @@ int launch_general(const bf16* q, size_t q_stride, const bf16* k, const bf16* vt
   if constexpr (D == 64 && NT == 4) {     // no variant with a sink or changed scores at this shape (its registers are spent)
     if (sink || extras) return MS_UNSUPPORTED;
   } else if (extras) {
-    if (extras->value_dim != D) {
-      if constexpr (VS == 1 && extra_variant<D, NT, WAVES, VS>()) {
-        attention_mfma_kernel<D, NT, WAVES, false, VS, true, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, nullptr, nullptr, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, pair_order, scan, sink, *extras);
-        return ms_launch_status();
-      } else {
-        return MS_UNSUPPORTED;
-      }
-    }
-    if constexpr (extra_variant<D, NT, WAVES, VS>()) {
-      attention_mfma_kernel<D, NT, WAVES, false, VS, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, nullptr, nullptr, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, pair_order, scan, sink, *extras);
-      return ms_launch_status();
-    } else {
+    const bool bounded = bounded_scores(*extras);
+    if constexpr (!extra_variant<D, NT, WAVES, VS>()) {
       return MS_UNSUPPORTED;
+    } else {
+#define LAUNCH_EXTRA(EX, NARROW) attention_mfma_kernel<D, NT, WAVES, false, VS, true, EX, NARROW><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, nullptr, nullptr, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, pair_order, scan, sink, *extras)
+      if (extras->value_dim != D) {
+        if constexpr (VS == 1) {
+          if (bounded) LAUNCH_EXTRA(BOUNDED, true); else LAUNCH_EXTRA(CHANGED, true);
+        } else {
+          return MS_UNSUPPORTED;
+        }
+      } else {
+        if (bounded) LAUNCH_EXTRA(BOUNDED, false); else LAUNCH_EXTRA(CHANGED, false);
+      }
+#undef LAUNCH_EXTRA
+      return ms_launch_status();
     }
   } else if (sink) {
     attention_mfma_kernel<D, NT, WAVES, false, VS, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, nullptr, nullptr, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, pair_order, scan, sink);
@@ -671,10 +764,13 @@ int launch_split(const bf16* q, size_t q_stride, const bf16* k, const bf16* vt, 
                  int n_requests, int nh, int nkv, int page_size, float scale, int window, int min_blocks,
                  int n_splits, const float* sink, const AttnExtras* extras, hipStream_t stream) {
   dim3 grid(n_splits, nkv, n_requests), block(4 * MS_WAVE);
-  if (extras && extras->value_dim != D)
-    attention_mfma_kernel<D, 1, 4, true, 1, true, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink, *extras);
-  else if (extras)
-    attention_mfma_kernel<D, 1, 4, true, 1, true, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink, *extras);
+#define LAUNCH_EXTRA(EX, NARROW) attention_mfma_kernel<D, 1, 4, true, 1, true, EX, NARROW><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink, *extras)
+  if (extras && extras->value_dim != D) {
+    if (bounded_scores(*extras)) LAUNCH_EXTRA(BOUNDED, true); else LAUNCH_EXTRA(CHANGED, true);
+  } else if (extras) {
+    if (bounded_scores(*extras)) LAUNCH_EXTRA(BOUNDED, false); else LAUNCH_EXTRA(CHANGED, false);
+  }
+#undef LAUNCH_EXTRA
   else if (sink)
     attention_mfma_kernel<D, 1, 4, true, 1, true><<<grid, block, 0, stream>>>(q, q_stride, k, vt, table, table_stride, table_rows, q_start, ctx, out, out_stride, part_o, part_ml, nh, nkv, page_size, page_shift_of(page_size), scale * 1.4426950408889634f, window, min_blocks, n_splits, sink);
   else
