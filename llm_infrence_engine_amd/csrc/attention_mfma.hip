@@ -122,10 +122,11 @@ __device__ __forceinline__ void load_values(ValueBlock<CT>& b, const bf16* __res
 // but only D / VS of the output's dims, so it reads all keys and 1 / VS of the values.  A compute unit draws
 // its data at a small fraction of the chip's rate, so when a step has fewer tiles than the chip has units this
 // shortens the longest chain without a second kernel; the blocks write disjoint dims and share nothing.
+//
 // EXTRA = CHANGED: the scores are changed on their way into the softmax: a scaled score x becomes cap * tanh(x / cap) (cap > 0),
 // then slope * (the key's distance from the query) is taken off it, one slope per query head; at the end every head's
-// result is multiplied by out_scale and by the sigmoid of a gate, one number per token and head or one per entry.  Such scores are kept
-// in log2 units from the start, and the block's maxima are those of the changed scores.
+// result is multiplied by out_scale and by the sigmoid of a gate, one number per token and head or one per entry.  Such
+// scores are kept in log2 units from the start, and the block's maxima are those of the changed scores.
 // EXTRA = BOUNDED: as CHANGED with a cap of at most BOUNDED_CAP and no slopes.  Such scores lie in [-cap, cap], whose
 // exponentials and their sums and products with values are well inside float's range, so the softmax needs no running
 // maximum: the reference stays where it starts (0; for the wave that holds a positive sink, the sink).
@@ -144,8 +145,8 @@ struct AttnExtras {
   int value_dim;             // the value size (NARROW variants: below the key size)
 };
 
-// The variants that change their scores need more registers than two wide tiles to a SIMD leave: a wide tile of theirs
-// has the SIMD to itself.  Narrow tiles over sixteen waves (128 registers a lane) and the narrow tile of the largest
+// The CHANGED variants need more registers than two wide tiles to a SIMD leave: a wide tile of theirs has the SIMD to
+// itself, as has a BOUNDED one with narrow values at the largest head size.  Narrow tiles over sixteen waves (128 registers a lane) and the narrow tile of the largest
 // head over eight have no such variant, nor have wide tiles over eight waves; the launcher picks a neighbour.
 template <int D, int NT, int WAVES, int VS>
 constexpr bool extra_variant() {
